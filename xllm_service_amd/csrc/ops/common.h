@@ -1,6 +1,6 @@
 // Common device helpers for the MI355X (gfx950 / CDNA4) kernels.
 //
-// Design notes (see /opt/skills/guides/cdna_hip_programming.md):
+// Design notes:
 //  * wavefront = 64 lanes; all block sizes are multiples of 64
 //  * bf16 global loads are vectorized as ushort4/ushort8 (8-16 B per lane)
 //  * fp32 accumulation everywhere; bf16 storage

@@ -141,28 +141,16 @@ class ModelRunner:
         enable, max_len, max_bs = self._graph_opts
         if not enable:
             return
-        from .graph_runner import DecodeGraphRunner, PrefillGraphRunner
+        from .graph_runner import DecodeGraphRunner
         self.graph_runner = DecodeGraphRunner(
             self.model, self.kv_caches, self.device,
             max_model_len=max_len, max_batch=max_bs)
         self.graph_runner.capture_all()
-        from xllm_service_amd.distributed import parallel_state as ps
         import os
-        # OPT-IN (XLLM_PREFILL_GRAPHS=1): replaying padded single-seq
-        # prefill chunks aborts with a device fault on the debug-model
-        # chunked-prefill shapes (L < bucket; tests/test_gpu_engine.py
-        # test_gpu_prefix_cache_and_chunked_prefill) while the full-length
-        # serving shape (L == 1024 == bucket) runs and saves ~2.5 ms per
-        # arrival. Until the padded-replay fault is isolated this stays
-        # off the default path — docs/TODO.md.
-        if (ps.tp_size() == 1
-                and os.environ.get("XLLM_PREFILL_GRAPHS") == "1"):
-            shared = os.environ.get("XLLM_PREFILL_GRAPH_SHARED_POOL") == "1"
-            self.prefill_graph = PrefillGraphRunner(
-                self.model, self.kv_caches, self.device,
-                max_model_len=max_len,
-                pool=self.graph_runner.pool if shared else None)
-            self.prefill_graph.capture_all()
+        # Replays of padded prompt chunks (L < bucket) aborted on the device
+        # and the cause is not known: prefill steps stay eager.
+        if os.environ.get("XLLM_PREFILL_GRAPHS") == "1":
+            raise RuntimeError("captured prefill steps are switched off")
 
     # ---- batch construction -------------------------------------------------
     def _build_batch(self, plan: StepPlan, bm):
