@@ -395,9 +395,8 @@ def test_expert_layer_every_execution_shape(target, T, identity, shared,
         m.router.copy_(w["l0.mlp.router"])
         m.correction.copy_(w["l0.mlp.correction"])
         for j in range(experts):
-            m.w_gate_up[j].copy_(torch.cat([w[f"l0.mlp.e{j}.gate"],
-                                            w[f"l0.mlp.e{j}.up"]]))
-            m.w_down[j].copy_(w[f"l0.mlp.e{j}.down"])
+            m.load_expert(j, w[f"l0.mlp.e{j}.up"], w[f"l0.mlp.e{j}.down"],
+                          w[f"l0.mlp.e{j}.gate"])
         if shared:
             m.shared_gate_up.copy_(torch.cat([w["l0.mlp.shared.gate"],
                                               w["l0.mlp.shared.up"]]))

@@ -438,14 +438,16 @@ def test_routed_experts_three_execution_shapes_agree(dev, skew):
         m.router.copy_(torch.randn(E, W, generator=g) * 0.5)
         if skew:
             m.router[0] += 3.0 * torch.ones(W) / math.sqrt(W)
-        m.w_gate_up.copy_(torch.randn(E, 2 * ff, W, generator=g) * 0.3)
-        m.w_down.copy_(torch.randn(E, W, ff, generator=g) * 0.3)
+        for e in range(E):
+            w1 = torch.randn(2 * ff, W, generator=g) * 0.3
+            m.load_expert(e, w1[ff:], torch.randn(W, ff, generator=g) * 0.3,
+                          gate=w1[:ff])
     h = torch.randn(T, W, generator=g) + (2.0 / math.sqrt(W) if skew else 0.0)
     wt = {"router": m.router.detach().to(F64)}
     for e in range(E):
-        wt[f"e{e}.gate"] = m.w_gate_up[e, :ff].detach().to(F64)
-        wt[f"e{e}.up"] = m.w_gate_up[e, ff:].detach().to(F64)
-        wt[f"e{e}.down"] = m.w_down[e].detach().to(F64)
+        wt[f"e{e}.gate"] = m.w_in[e, :, :ff].t().detach().to(F64)
+        wt[f"e{e}.up"] = m.w_in[e, :, ff:].t().detach().to(F64)
+        wt[f"e{e}.down"] = m.w_down[e].t().detach().to(F64)
     fc = dict(router=dict(experts=E, top=top, groups=dict(count=4, keep=2)))
     want = o_experts(wt, "", fc, h.to(F64))
     m = m.to(dev)

@@ -10,7 +10,7 @@ from typing import List, Optional
 @dataclass
 class ModelConfig:
     name: str = "llama"
-    architecture: str = "llama"   # llama | opt | qwen2 | qwen2_vl | pugovik | dunusun | tosipel | gararax
+    architecture: str = "llama"   # llama | opt | qwen2 | qwen2_vl | pugovik | dunusun | tosipel | gararax | nikedra
     vocab_size: int = 128256
     hidden_size: int = 4096
     intermediate_size: int = 14336
@@ -339,6 +339,50 @@ def gararax_from_dict(d: dict, name: str = "gararax",
         max_position=1 << 20, layers=layers, model_dir=model_dir)
 
 
+@dataclass
+class NikedraConfig(ModelConfig):
+    """Nikedra: layers of windowed latent attention (`latent_attention`), a
+    delta rule with one decay per key channel (`channel_delta`), or chunked
+    softmax attention beside a selective state space mixer (`parallel`, each
+    half normed); mixer and feed-forward read the same residual through two
+    norms of one number each, the mixer behind a short convolution; dense
+    clamped-gate or routed-expert feed-forwards (the router weight on the
+    expert's input); after every layer the residual becomes a weighted sum
+    of the embedding and all layer results so far."""
+    layers: List[HybridLayerConfig] = field(default_factory=list)
+    canon_taps: int = 1                 # input convolution of every mixer
+    logit_scale: float = 1.0
+    model_dir: Optional[str] = None     # weights live here (None = random)
+
+    @property
+    def has_recurrent_state(self) -> bool:
+        return True
+
+
+NIKEDRA_MIXERS = ("latent_attention", "channel_delta", "parallel")
+
+
+def nikedra_from_dict(d: dict, name: str = "nikedra",
+                      model_dir: Optional[str] = None) -> NikedraConfig:
+    layers = [HybridLayerConfig(type=l["type"], mixer=dict(l["mixer"]),
+                                mlp=l.get("mlp"))
+              for l in d["layers"]]
+    for i, l in enumerate(layers):
+        if l.type not in NIKEDRA_MIXERS:
+            raise ValueError(f"layer {i}: unknown mixer type {l.type!r}")
+        if l.mlp is not None and l.mlp.get("kind") not in ("dense", "moe"):
+            raise ValueError(f"layer {i}: unknown feed-forward kind")
+    taps = int((d.get("canon") or {}).get("taps", 1))
+    if taps < 1:
+        raise ValueError("canon: taps must be >= 1")
+    return NikedraConfig(
+        name=name, architecture="nikedra", vocab_size=int(d["vocab"]),
+        hidden_size=int(d["width"]), num_layers=len(layers),
+        rms_eps=float(d["norm"]["eps"]), canon_taps=taps,
+        logit_scale=float(d.get("logit_scale", 1.0)),
+        max_position=1 << 20, layers=layers, model_dir=model_dir)
+
+
 def load_model_dir(path: str) -> ModelConfig:
     """Read <path>/config.json and pick the config class by its
     `architecture` field."""
@@ -357,6 +401,9 @@ def load_model_dir(path: str) -> ModelConfig:
     if arch == "gararax":
         return gararax_from_dict(d, name=os.path.basename(
             os.path.normpath(path)) or "gararax", model_dir=path)
+    if arch == "nikedra":
+        return nikedra_from_dict(d, name=os.path.basename(
+            os.path.normpath(path)) or "nikedra", model_dir=path)
     raise ValueError(f"{path}: unsupported architecture "
                      f"{d.get('architecture')!r}")
 
@@ -552,6 +599,58 @@ PRESETS.update({
     # bench stacks at the width of real deployments (random weights)
     "gararax-2k": _gararax_preset("gararax-2k", 2048, 8),
     "gararax-4k": _gararax_preset("gararax-4k", 4096, 8),
+})
+
+
+def _nikedra_preset(name, width, n_layers, vocab=32000, head=128, window=1024,
+                    kv_rank=512, rot_dim=64, experts=16, top=2, state=128,
+                    rank=64):
+    """Synthetic Nikedra stacks for benchmarks: per group of four layers two
+    channel-decay delta layers, one parallel layer (chunked attention beside
+    a state space mixer) and one windowed latent attention layer; dense and
+    routed feed-forwards in turn."""
+    heads = max(width // head, 1)
+    dense = dict(kind="dense", ff=3 * width // 2, limit=7.0)
+    moe = dict(kind="moe", expert=dict(ff=width // 2),
+               router=dict(experts=experts, top=top))
+    layers = []
+    for i in range(n_layers):
+        k, mlp = i % 4, moe if i % 2 else dense
+        if k == 1:
+            sh = max(width // (head // 2), 1)
+            layers.append(dict(type="parallel", mlp=mlp, mixer=dict(
+                left=dict(heads=heads, kv_heads=max(heads // 4, 1), dim=head,
+                          vdim=head, mask=dict(size=window),
+                          scale=head ** -0.5,
+                          rot=dict(base=10000.0, dims=head // 2, scaling=dict(
+                              factor=4.0, fast=32.0, original=4096,
+                              slow=1.0))),
+                right=dict(heads=sh, vdim=head // 2, state=state,
+                           groups=max(sh // 4, 1),
+                           norm_groups=max(sh // 4, 1), conv=4))))
+        elif k == 3:
+            layers.append(dict(type="latent_attention", mlp=mlp, mixer=dict(
+                heads=heads, dim=head, rot_dim=rot_dim, vdim=head,
+                kv_rank=kv_rank, mask=dict(size=window),
+                scale=(head + rot_dim) ** -0.5,
+                rot=dict(base=10000.0, dims=rot_dim))))
+        else:
+            layers.append(dict(type="channel_delta", mlp=mlp, mixer=dict(
+                heads=heads, kv_heads=max(heads // 2, 1), dim=head, vdim=head,
+                conv=4, decay_rank=rank, gate_rank=rank)))
+    return nikedra_from_dict(dict(
+        architecture="Nikedra", vocab=vocab, width=width, layers=layers,
+        norm=dict(eps=1e-6), canon=dict(taps=4), logit_scale=0.5), name=name)
+
+
+PRESETS.update({
+    # CPU-test sized stack
+    "nikedra-tiny": _nikedra_preset("nikedra-tiny", 64, 4, vocab=256, head=16,
+                                    window=20, kv_rank=24, rot_dim=8,
+                                    experts=6, top=2, state=8, rank=6),
+    # bench stacks at the width of real deployments (random weights)
+    "nikedra-2k": _nikedra_preset("nikedra-2k", 2048, 8),
+    "nikedra-4k": _nikedra_preset("nikedra-4k", 4096, 8),
 })
 
 

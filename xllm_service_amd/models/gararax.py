@@ -234,12 +234,10 @@ class GararaxForCausalLM(nn.Module):
                     put(ff.router, take(f + "router"))
                     if f + "correction" in tensors:
                         put(ff.correction, take(f + "correction"))
-                    put(ff.w_gate_up, torch.stack([
-                        torch.cat([take(f"{f}e{j}.gate"),
-                                   take(f"{f}e{j}.up")], 0)
-                        for j in range(ff.experts)]))
-                    put(ff.w_down, torch.stack([take(f"{f}e{j}.down")
-                                                for j in range(ff.experts)]))
+                    for j in range(ff.experts):
+                        e = f"{f}e{j}."
+                        ff.load_expert(j, take(e + "up"), take(e + "down"),
+                                       take(e + "gate"))
                     if ff.shared_ff:
                         put(ff.shared_gate_up,
                             torch.cat([take(f + "shared.gate"),
@@ -280,7 +278,8 @@ class GararaxForCausalLM(nn.Module):
                 elif leaf == "weight":                 # embedding tables
                     p.copy_(randn(p.shape).to(p.dtype))
                 else:
-                    std = 1.0 / math.sqrt(p.shape[-1])
+                    # expert matrices are kept [expert, in, out]
+                    std = 1.0 / math.sqrt(p.shape[-2 if p.dim() == 3 else -1])
                     p.copy_((randn(p.shape) * std).to(p.dtype))
 
     # ---- forward -----------------------------------------------------------

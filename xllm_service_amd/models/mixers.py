@@ -36,8 +36,11 @@ GroupedAttention       softmax attention with grouped key/value heads whose
                        the half layout (plain or with banded frequency
                        scaling), unit RMS norm of q and k per head after the
                        turn, a sliding window that also keeps the first
-                       tokens, a sink of score 0, one score multiplier per
-                       head, keys read as values, element-wise sigmoid gate.
+                       tokens, chunks instead of a window, a sink of score 0,
+                       one score multiplier per head, keys read as values,
+                       sigmoid gate per element or per head.
+InputConvolution       h + causal convolution of h over time, in front of a
+                       mixer's projections.
 
 All take the slice of a merged input projection that belongs to them and
 return the mixer output in the model dtype. Sizes and constants are
@@ -111,13 +114,17 @@ class LatentAttention(nn.Module):
     """rot None (with rot_dim 0): no rotated key part, no positions.
     q_rank: the queries come from a normed low-rank latent of that size
     (the merged projection then holds the latent's rows instead of q).
-    gated False: no sigmoid output gate."""
+    gated False: no sigmoid output gate. window > 0: a query sees the last
+    `window` keys. rot_pairs: entries (2i, 2i+1) turn together, else
+    (i, i + dims/2)."""
 
     def __init__(self, width: int, heads: int, dim: int, rot_dim: int,
                  vdim: int, kv_rank: int, scale: float, rot: Optional[dict],
                  norm_eps: float, kv_from: Optional[int], dtype,
-                 q_rank: Optional[int] = None, gated: bool = True):
+                 q_rank: Optional[int] = None, gated: bool = True,
+                 window: int = 0, rot_pairs: bool = True):
         super().__init__()
+        self.window, self.rot_pairs = int(window), bool(rot_pairs)
         self.heads, self.dim, self.rot_dim = heads, dim, rot_dim
         self.vdim, self.kv_rank = vdim, kv_rank
         self.scale, self.eps, self.kv_from = float(scale), norm_eps, kv_from
@@ -168,12 +175,12 @@ class LatentAttention(nn.Module):
             q = proj[:, :self.q_width].unflatten(-1, (H, dim + rd))
         if self.rot_dims:
             hops.rope_interleaved_(q, positions, self.inv_freq, self.mscale,
-                                   dim, self.rot_dims)
+                                   dim, self.rot_dims, self.rot_pairs)
         if self.kv_from is None:
             dkv = proj[:, self.q_in:self.q_in + self.dkv_width]
             hops.latent_kv_store(dkv, self.dkv_norm, self.eps, positions,
                                  self.inv_freq, self.mscale, self.rot_dims,
-                                 cache, meta.slot_mapping, r)
+                                 cache, meta.slot_mapping, r, self.rot_pairs)
         # fold the queries through the key up-projection: [H,T,dim]x[H,dim,r]
         q_abs = torch.bmm(q[..., :dim].transpose(0, 1), self.w_uk)
         if rd:
@@ -188,10 +195,11 @@ class LatentAttention(nn.Module):
         if np_:
             hops.latent_attn(qf[:np_], cache, meta.prefill_block_tables,
                              meta.cu_q, meta.prefill_seq_lens, self.scale, r,
-                             lat[:np_])
+                             lat[:np_], self.window)
         if nd:
             hops.latent_attn(qf[np_:], cache, meta.decode_block_tables, None,
-                             meta.decode_seq_lens, self.scale, r, lat[np_:])
+                             meta.decode_seq_lens, self.scale, r, lat[np_:],
+                             self.window)
         # value up-projection per head: [H,T,r] x [H,r,vdim]
         o = torch.bmm(lat.to(proj.dtype).transpose(0, 1), self.w_uv_t)
         o = o.transpose(0, 1).reshape(T, H * self.vdim)
@@ -261,6 +269,27 @@ def _halves(meta: AttnMetadata, aux):
     return out
 
 
+class InputConvolution(nn.Module):
+    """h + conv(h), a causal convolution over time with one filter per
+    channel; the sequence's last taps - 1 inputs are carried."""
+
+    def __init__(self, width: int, taps: int, dtype):
+        super().__init__()
+        self.width, self.taps = width, taps
+        self.w = nn.Parameter(torch.empty(width, taps, dtype=dtype))
+
+    def cache_spec(self):
+        return ConvState(self.width, self.taps)
+
+    def forward(self, h, state, meta: AttnMetadata, aux):
+        out = torch.empty_like(h)
+        for rows, cu_q, ctx, slots, _, _, _ in _halves(meta, aux):
+            hops.short_conv(h[rows], self.w, None, state, 0, slots, cu_q, ctx,
+                            1, self.width, add_input=True, advance=True,
+                            out=out[rows])
+        return out
+
+
 class SelectiveStateSpace(nn.Module):
     """in_proj rows: [z: inner | x: inner | B: G*N | C: G*N | dt: heads],
     inner = heads * vdim."""
@@ -302,8 +331,7 @@ class SelectiveStateSpace(nn.Module):
             u = xbc_in[rows]
             xbc = hops.short_conv(u, self.conv_w, self.conv_b, conv_state, 0,
                                   slots, cu_q, ctx, 1, self.conv_ch,
-                                  act_silu=True)
-            hops.short_conv_state_(conv_state, u, slots, cu_q)
+                                  act_silu=True, advance=True)
             hops.gated_recurrence(
                 0, xbc[:, inner + gn:], xbc[:, inner:inner + gn],
                 xbc[:, :inner], dt[rows], self.dt_bias, self.A_log, self.D,
@@ -424,11 +452,18 @@ class GatedLinearAttention(nn.Module):
 
 class ParallelMixer(nn.Module):
     """Two mixers on the same input; the caller adds their outputs with the
-    weights `scales` (kept apart so the sum is taken in fp32)."""
+    weights `scales` (kept apart so the sum is taken in fp32). normed: the
+    caller also divides each by its root mean square over that many columns,
+    times left_norm / right_norm."""
 
     def __init__(self, left: nn.Module, right: nn.Module, left_scale: float,
-                 right_scale: float):
+                 right_scale: float, normed: Optional[int] = None):
         super().__init__()
+        if normed:
+            self.left_norm = nn.Parameter(torch.ones(normed,
+                                                     dtype=torch.float32))
+            self.right_norm = nn.Parameter(torch.ones(normed,
+                                                      dtype=torch.float32))
         self.left, self.right = left, right
         self.scales = (float(left_scale), float(right_scale))
         self.in_width = left.in_width + right.in_width
@@ -502,10 +537,17 @@ class SinkWindowAttention(nn.Module):
 class GatedDeltaRule(nn.Module):
     """in_proj rows: [q: kv_heads*dim | k: kv_heads*dim | v: heads*vdim |
     g: heads*vdim | b: heads | a: heads]; q, k, v pass the short
-    convolution (filters stacked in that order) and SiLU."""
+    convolution (filters stacked in that order) and SiLU.
+
+    decay_rank: one decay per head and KEY CHANNEL, from a low-rank
+    projection a2 (a1 h) of that inner size; gate_rank: the output gate is
+    g2 (g1 h) of that inner size. The rows of g and a are then those of g1
+    and a1. gate_silu False: sigmoid gate."""
 
     def __init__(self, width: int, heads: int, kv_heads: int, dim: int,
-                 vdim: int, taps: int, norm_eps: float, dtype):
+                 vdim: int, taps: int, norm_eps: float, dtype, *,
+                 decay_rank: Optional[int] = None,
+                 gate_rank: Optional[int] = None, gate_silu: bool = True):
         super().__init__()
         if heads % kv_heads:
             raise ValueError("heads must be a multiple of kv_heads")
@@ -514,10 +556,21 @@ class GatedDeltaRule(nn.Module):
         self.taps, self.eps = taps, norm_eps
         self.qk_width, self.v_width = kv_heads * dim, heads * vdim
         self.conv_ch = 2 * self.qk_width + self.v_width
-        self.in_width = self.conv_ch + self.v_width + 2 * heads
+        self.decay_rank, self.gate_rank = decay_rank, gate_rank
+        self.gate_silu = gate_silu
+        self.g_in = gate_rank or self.v_width
+        self.a_in = decay_rank or heads
+        self.in_width = self.conv_ch + self.g_in + heads + self.a_in
         f32 = dict(dtype=torch.float32)
         self.conv_w = nn.Parameter(torch.empty(self.conv_ch, taps, dtype=dtype))
-        self.dt_bias = nn.Parameter(torch.zeros(heads, **f32))
+        n_decay = heads * (dim if decay_rank else 1)
+        if decay_rank:
+            self.a2 = nn.Parameter(torch.empty(n_decay, decay_rank,
+                                               dtype=dtype))
+        if gate_rank:
+            self.g2 = nn.Parameter(torch.empty(self.v_width, gate_rank,
+                                               dtype=dtype))
+        self.dt_bias = nn.Parameter(torch.zeros(n_decay, **f32))
         self.A_log = nn.Parameter(torch.zeros(heads, **f32))
         self.out_norm = nn.Parameter(torch.ones(vdim, **f32))
         self.o_proj = nn.Parameter(torch.empty(width, self.v_width,
@@ -532,28 +585,33 @@ class GatedDeltaRule(nn.Module):
         T, a, b, H = proj.shape[0], self.qk_width, self.v_width, self.heads
         c = self.conv_ch
         u_all = proj[:, :c]
-        gate = proj[:, c:c + b]
-        beta, dt = proj[:, c + b:c + b + H], proj[:, c + b + H:self.in_width]
+        e = c + self.g_in
+        gate, beta = proj[:, c:e], proj[:, e:e + H]
+        dt = proj[:, e + H:self.in_width]
+        if self.gate_rank:
+            gate = F.linear(gate, self.g2)
+        if self.decay_rank:
+            dt = F.linear(dt, self.a2)
         o = torch.empty(T, H, self.vdim, dtype=torch.float32,
                         device=proj.device)
         for rows, cu_q, ctx, slots, _, _, max_len in _halves(meta, aux):
             u = u_all[rows]
             x = hops.short_conv(u, self.conv_w, None, conv_state, 0, slots,
-                                cu_q, ctx, 1, c, act_silu=True)
-            hops.short_conv_state_(conv_state, u, slots, cu_q)
+                                cu_q, ctx, 1, c, act_silu=True, advance=True)
             hops.delta_rule(x[:, :a], x[:, a:2 * a], x[:, 2 * a:], beta[rows],
                             dt[rows], self.dt_bias, self.A_log, state, slots,
                             cu_q, ctx, self.kv_heads, o[rows],
                             max_q_len=max_len)
         y = hops.gated_group_norm(o.view(T, b), self.out_norm, gate, self.eps,
-                                  H, act_silu=True, gate_first=False,
-                                  out_dtype=proj.dtype)
+                                  H, act_silu=self.gate_silu,
+                                  gate_first=False, out_dtype=proj.dtype)
         return F.linear(y, self.o_proj)
 
 
 class GroupedAttention(nn.Module):
     """in_proj rows: [q: heads*dim | k: kv_heads*dim | v: kv_heads*vdim
-    (absent with values_are_keys) | g: heads*vdim (with gated)].
+    (absent with values_are_keys) | g: heads*vdim (with gated), heads (with
+    head_gated)].
 
     rot: {base, dims, scaling?} or None; rot_pairs: entries (2i, 2i+1) turn
     together, else (i, i + dims/2). unit_norm: q and k are divided by their
@@ -561,14 +619,19 @@ class GroupedAttention(nn.Module):
     keep_first: the first keys stay visible beside the window. zero_sink: 1
     joins the softmax denominator. head_scale: a learned score multiplier
     per head. values_are_keys: the weighted sum runs over the cached keys.
-    gated: the heads' outputs are multiplied by sigmoid(g)."""
+    gated: the heads' outputs are multiplied by sigmoid(g); head_gated: by
+    one such number per head. chunked: `window` is the size of the chunks,
+    counted from position 0, that keep to themselves. yarn: rot's `scaling`
+    is that of scaled_rope_frequencies (ramp over the pair index, cos/sin
+    multiplier), else that of banded_rope_frequencies."""
 
     def __init__(self, width: int, heads: int, kv_heads: int, dim: int,
                  vdim: int, rot: Optional[dict], rot_pairs: bool,
                  scale: float, window: int, keep_first: int, norm_eps: float,
                  dtype, *, unit_norm: bool = False, zero_sink: bool = False,
                  head_scale: bool = False, values_are_keys: bool = False,
-                 gated: bool = False):
+                 gated: bool = False, head_gated: bool = False,
+                 chunked: bool = False, yarn: bool = False):
         super().__init__()
         if heads % kv_heads:
             raise ValueError("heads must be a multiple of kv_heads")
@@ -579,16 +642,25 @@ class GroupedAttention(nn.Module):
         self.scale, self.eps = float(scale), norm_eps
         self.window, self.keep_first = int(window), int(keep_first)
         self.rot_pairs, self.unit_norm = bool(rot_pairs), bool(unit_norm)
-        self.values_are_keys, self.gated = values_are_keys, gated
+        self.values_are_keys = values_are_keys
+        self.gated, self.chunked = gated or head_gated, bool(chunked)
+        if gated and head_gated:
+            raise ValueError("one kind of output gate")
         self.rot_dims = int(rot["dims"]) if rot else 0
         if self.rot_dims > dim or self.rot_dims % 2:
             raise ValueError("rotary dims must be even and <= dim")
-        inv_freq = banded_rope_frequencies(rot) if self.rot_dims \
-            else torch.zeros(0, dtype=torch.float64)
+        self.mscale = 1.0
+        if not self.rot_dims:
+            inv_freq = torch.zeros(0, dtype=torch.float64)
+        elif yarn:
+            inv_freq, self.mscale = scaled_rope_frequencies(rot)
+        else:
+            inv_freq = banded_rope_frequencies(rot)
         self.register_buffer("inv_freq", inv_freq, persistent=False)
         self.cq, self.ck = heads * dim, kv_heads * dim
         self.cv = 0 if values_are_keys else kv_heads * vdim
-        self.g_width = heads * vdim if gated else 0
+        self.gate_cols = vdim if head_gated else 1   # columns per gate entry
+        self.g_width = heads * vdim // self.gate_cols if self.gated else 0
         self.in_width = self.cq + self.ck + self.cv + self.g_width
         f32 = dict(dtype=torch.float32)
         if zero_sink:
@@ -613,7 +685,7 @@ class GroupedAttention(nn.Module):
         q = hops.rope_headnorm_store(
             proj[:, :cq], proj[:, cq:cq + ck], v_in, positions, self.inv_freq,
             self.rot_dims, self.rot_pairs, self.unit_norm, self.eps, H,
-            self.kv_heads, k_cache, v_cache, meta.slot_mapping)
+            self.kv_heads, k_cache, v_cache, meta.slot_mapping, self.mscale)
         o = torch.empty(T, H, self.vdim, dtype=torch.float32,
                         device=proj.device)
         for rows, cu_q, _, _, seq_lens, tables, _ in _halves(meta, aux):
@@ -621,11 +693,13 @@ class GroupedAttention(nn.Module):
                              seq_lens, H, self.scale, 0.0, o[rows],
                              window=self.window, sink=self.sink,
                              keep_first=self.keep_first,
-                             head_scale=self.head_scale)
+                             head_scale=self.head_scale,
+                             chunked=self.chunked)
         o = o.view(T, H * self.vdim)
         if self.gated:
             y = hops.norm_sigmoid_gate(
-                o, None, proj[:, cq + ck + cv:self.in_width], 0.0, proj.dtype)
+                o, None, proj[:, cq + ck + cv:self.in_width], 0.0, proj.dtype,
+                gate_cols=self.gate_cols)
         else:
             y = o.to(proj.dtype)
         return F.linear(y, self.o_proj)

@@ -9,8 +9,14 @@ matrix per expert.
 Options: softmax scores over all experts, a correction added to the scores
 for the choice only, groups scored by their best expert, weights divided by
 their sum, `identity` further router outputs that stand for experts without
-tensors whose output is their input, and a shared expert of the same form
-that every token uses (added to the routed sum in fp32).
+tensors whose output is their input, a shared expert of the same form that
+every token uses (added to the routed sum in fp32), experts without a gate
+(down(gelu(up h)), exact GELU), and the router weight on an expert's input
+instead of its output (the up-projection is linear, so the activation kernel
+applies the weight to its rows).
+
+Expert matrices are kept [expert, in, out], the contiguous right operand of a
+batched product.
 
 Two execution shapes over the same weights, both ending in the fp32 combine
 kernel: few tokens (decode batches, graph capture) run every expert as one
@@ -34,7 +40,8 @@ class RoutedExperts(nn.Module):
                  n_groups: int, keep: int, dtype, dense_max_tokens: int = 64,
                  *, identity: int = 0, softmax: bool = False,
                  correction: bool = False, group_max: bool = False,
-                 normalize: bool = False, shared_ff: int = 0):
+                 normalize: bool = False, shared_ff: int = 0,
+                 gated: bool = True, weight_input: bool = False):
         super().__init__()
         n_all = experts + identity
         if n_all % n_groups or keep > n_groups or \
@@ -44,14 +51,18 @@ class RoutedExperts(nn.Module):
         self.n_groups, self.keep = n_groups, keep
         self.identity, self.softmax = identity, softmax
         self.group_max, self.normalize = group_max, normalize
+        if weight_input and (gated or identity or shared_ff):
+            raise ValueError("weights on the input: plain experts only")
+        self.gated, self.weight_input = gated, weight_input
         self.dense_max_tokens = dense_max_tokens
         self.router = nn.Parameter(torch.empty(n_all, width,
                                                dtype=torch.float32))
         self.correction = nn.Parameter(torch.zeros(
             n_all, dtype=torch.float32)) if correction else None
-        self.w_gate_up = nn.Parameter(torch.empty(experts, 2 * ff, width,
-                                                  dtype=dtype))
-        self.w_down = nn.Parameter(torch.empty(experts, width, ff,
+        # columns [gate | up] (up alone without a gate)
+        self.w_in = nn.Parameter(torch.empty(
+            experts, width, (2 if gated else 1) * ff, dtype=dtype))
+        self.w_down = nn.Parameter(torch.empty(experts, ff, width,
                                                dtype=dtype))
         self.shared_ff = shared_ff
         if shared_ff:
@@ -59,6 +70,21 @@ class RoutedExperts(nn.Module):
                 2 * shared_ff, width, dtype=dtype))
             self.shared_down = nn.Parameter(torch.empty(width, shared_ff,
                                                         dtype=dtype))
+
+    def load_expert(self, e: int, up, down, gate=None) -> None:
+        """Checkpoint tensors [out, in] of expert e."""
+        w_in = up if gate is None else torch.cat([gate, up], 0)
+        with torch.no_grad():
+            for p, w in ((self.w_in[e], w_in), (self.w_down[e], down)):
+                if tuple(w.t().shape) != tuple(p.shape):
+                    raise ValueError(f"expert {e}: shape mismatch "
+                                     f"{tuple(w.shape)}")
+                p.copy_(w.t().to(p.dtype))
+
+    def _act(self, z, scale=None, ids=None, wts=None):
+        if self.gated:
+            return hops.silu_mul(z)
+        return hops.gelu_scaled(z, scale, ids, wts)
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         """h [T, width] (model dtype) -> fp32 [T, width]."""
@@ -72,16 +98,19 @@ class RoutedExperts(nn.Module):
             extra = F.linear(hops.silu_mul(F.linear(h, self.shared_gate_up)),
                              self.shared_down)
         ident = h if self.identity else None
+        win = self.weight_input
+        mix = None if win else wts         # what the combine multiplies by
         capturing = h.is_cuda and torch.cuda.is_current_stream_capturing()
         if T <= self.dense_max_tokens or capturing:
-            gu = torch.matmul(h, self.w_gate_up.transpose(1, 2))  # [E,T,2ff]
-            act = hops.silu_mul(gu)
-            y = torch.bmm(act, self.w_down.transpose(1, 2))       # [E,T,W]
+            z = torch.bmm(h.expand(E, T, -1), self.w_in)     # [E, T, (2)ff]
+            act = self._act(z, None, ids if win else None,
+                            wts if win else None)
+            y = torch.bmm(act, self.w_down)                  # [E, T, W]
             rows = ids * T + torch.arange(T, dtype=torch.int32,
                                           device=h.device)[:, None]
             if self.identity:
                 rows = torch.where(ids >= E, -1, rows)
-            return hops.moe_combine(y, rows, wts, T, ident, extra)
+            return hops.moe_combine(y, rows, mix, T, ident, extra)
         # identity choices sort behind every expert and take no rows
         flat = ids.reshape(-1).long()
         order = torch.argsort(flat, stable=True)
@@ -95,8 +124,9 @@ class RoutedExperts(nn.Module):
                           device=h.device)
         if total == 0:
             y = h.new_zeros(1, self.width)
-            return hops.moe_combine(y, rows.view(T, self.top), wts, T, ident,
+            return hops.moe_combine(y, rows.view(T, self.top), mix, T, ident,
                                     extra)
+        scale = wts.reshape(-1)[order] if win else None      # per sorted row
         if cap * E <= 1.5 * total + 16 * E:
             # near-even load: pad every expert to `cap` rows and run all of
             # them as two batched GEMMs
@@ -106,12 +136,13 @@ class RoutedExperts(nn.Module):
                                      - starts[e_sorted])
             xs = h.new_zeros(E * cap, self.width)
             xs[dest] = h[order // self.top]
-            gu = torch.bmm(xs.view(E, cap, self.width),
-                           self.w_gate_up.transpose(1, 2))
-            y = torch.bmm(hops.silu_mul(gu), self.w_down.transpose(1, 2))
+            if win:
+                scale = scale.new_zeros(E * cap).index_copy_(0, dest, scale)
+            z = torch.bmm(xs.view(E, cap, self.width), self.w_in)
+            y = torch.bmm(self._act(z, scale), self.w_down)
             rows[order] = dest.to(torch.int32)
             return hops.moe_combine(y.view(-1, self.width),
-                                    rows.view(T, self.top), wts, T, ident,
+                                    rows.view(T, self.top), mix, T, ident,
                                     extra)
         xs = h[order // self.top]
         ys = torch.empty(total, self.width, dtype=h.dtype, device=h.device)
@@ -119,9 +150,10 @@ class RoutedExperts(nn.Module):
         for e, n in enumerate(counts):
             if n:
                 seg = slice(at, at + n)
-                act = hops.silu_mul(F.linear(xs[seg], self.w_gate_up[e]))
-                ys[seg] = F.linear(act, self.w_down[e])
+                act = self._act(xs[seg] @ self.w_in[e],
+                                scale[seg] if win else None)
+                ys[seg] = act @ self.w_down[e]
                 at += n
         rows[order] = torch.arange(total, dtype=torch.int32, device=h.device)
-        return hops.moe_combine(ys, rows.view(T, self.top), wts, T, ident,
+        return hops.moe_combine(ys, rows.view(T, self.top), mix, T, ident,
                                 extra)

@@ -153,12 +153,10 @@ class PugovikForCausalLM(nn.Module):
             if layer.mlp is not None:
                 e = layer.mlp
                 put(e.router, take(p + "mlp.router"))
-                put(e.w_gate_up, torch.stack([
-                    torch.cat([take(f"{p}mlp.e{j}.gate"),
-                               take(f"{p}mlp.e{j}.up")], 0)
-                    for j in range(e.experts)]))
-                put(e.w_down, torch.stack([take(f"{p}mlp.e{j}.down")
-                                           for j in range(e.experts)]))
+                for j in range(e.experts):
+                    q = f"{p}mlp.e{j}."
+                    e.load_expert(j, take(q + "up"), take(q + "down"),
+                                  take(q + "gate"))
                 put(layer.rg2, take(p + "rg2"))
                 put(layer.rg2_b, take(p + "rg2.b"))
                 for n in ("norm2", "norm2b", "ls2"):
@@ -179,7 +177,9 @@ class PugovikForCausalLM(nn.Module):
                         p.copy_(1.0 + 0.1 * torch.randn(
                             p.shape, generator=gen, device=dev))
                     continue
-                std = 1.0 / math.sqrt(p.shape[-1])
+                # expert matrices are kept [expert, in, out]
+                std = 1.0 / math.sqrt(p.shape[-2 if p.dim() == 3
+                                              and ".mlp." in name else -1])
                 p.copy_((torch.randn(p.shape, generator=gen, device=dev,
                                      dtype=torch.float32) * std).to(p.dtype))
 

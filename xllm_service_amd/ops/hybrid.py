@@ -2,7 +2,7 @@
 recurrent state, grouped RMS norms, gated residuals, routed experts;
 residual streams, short convolutions, gated recurrences, soft-capped and
 windowed paged attention; post-norm residual, whole-row q/k norm with
-rotate-half positions, the gated delta rule.
+rotate-half positions, the gated delta rule; depth average of the residual.
 
 Same policy as the rest of `ops`: on a GPU the HIP extension (`_ops_hybrid`)
 is the only path and its absence raises; on CPU the fp32 torch references in
@@ -78,36 +78,41 @@ def silu_mul(x):
 
 
 def rope_interleaved_(x, positions, inv_freq, mscale: float, off: int,
-                      rot_dims: int):
-    """Rotate x[..., off:off+rot_dims] ([T, H, D] view) in place."""
+                      rot_dims: int, pairs: bool = True):
+    """Rotate x[..., off:off+rot_dims] ([T, H, D] view) in place; pairs
+    False: entry i turns with entry i + rot_dims/2."""
     if x.is_cuda:
-        _hyb().rope_interleaved(x, positions, inv_freq, mscale, off, rot_dims)
+        _hyb().rope_interleaved(x, positions, inv_freq, mscale, off, rot_dims,
+                                pairs)
         return x
     x[..., off:off + rot_dims] = ref.rope_interleaved(
-        x[..., off:off + rot_dims], positions, inv_freq, mscale, rot_dims)
+        x[..., off:off + rot_dims], positions, inv_freq, mscale, rot_dims,
+        pairs)
     return x
 
 
 def latent_kv_store(dkv, norm_w, eps, positions, inv_freq, mscale, rot_dims,
-                    cache, slot_mapping, kv_rank):
+                    cache, slot_mapping, kv_rank, pairs: bool = True):
     if dkv.is_cuda:
         _hyb().latent_kv_store(cache, dkv, norm_w, eps, positions, inv_freq,
-                               mscale, rot_dims, slot_mapping, kv_rank)
+                               mscale, rot_dims, slot_mapping, kv_rank, pairs)
         return
     ref.latent_kv_store(dkv, norm_w, eps, positions, inv_freq, mscale,
-                        rot_dims, cache, slot_mapping, kv_rank)
+                        rot_dims, cache, slot_mapping, kv_rank, pairs)
 
 
-def latent_attn(q, cache, block_tables, cu_q, seq_lens, scale, kv_rank, out):
-    """out fp32 [T, H, kv_rank] (written). cu_q None: decode rows."""
+def latent_attn(q, cache, block_tables, cu_q, seq_lens, scale, kv_rank, out,
+                window: int = 0):
+    """out fp32 [T, H, kv_rank] (written). cu_q None: decode rows. window > 0
+    limits a query to the last `window` keys (itself included)."""
     if q.is_cuda:
         _hyb().latent_attn(out, q, cache, block_tables, cu_q, seq_lens, scale,
-                           kv_rank)
+                           kv_rank, window)
         return out
     if cu_q is None:
         cu_q = torch.arange(q.shape[0] + 1, dtype=torch.int32)
     out.copy_(ref.latent_attn(q, cache, block_tables, cu_q, seq_lens, scale,
-                              kv_rank))
+                              kv_rank, window))
     return out
 
 
@@ -153,7 +158,8 @@ def moe_route(h, w_router, top: int, n_groups: int, keep: int, *,
 
 def moe_combine(y, rows, wts, tokens: int, ident=None, extra=None):
     """fp32 [tokens, width] = sum_k wts[t, k] * y[rows[t, k]] (+ extra[t]).
-    A negative row stands for the token's own input: ident[t]."""
+    A negative row stands for the token's own input: ident[t]. wts None:
+    plain sum."""
     width = y.shape[-1]
     if y.is_cuda:
         out = torch.empty(tokens, width, dtype=torch.float32, device=y.device)
@@ -162,7 +168,7 @@ def moe_combine(y, rows, wts, tokens: int, ident=None, extra=None):
     yy = y.reshape(-1, width).float()[rows.long().clamp(min=0)]   # [T,top,W]
     if ident is not None:
         yy = torch.where((rows < 0)[:, :, None], ident.float()[:, None, :], yy)
-    out = (yy * wts[:, :, None]).sum(1)
+    out = yy.sum(1) if wts is None else (yy * wts[:, :, None]).sum(1)
     return out if extra is None else out + extra.float()
 
 
@@ -223,21 +229,37 @@ def softcap(x, cap: float):
 def short_conv(x, w, bias, state, state_off: int, slots, cu_q, ctx_lens,
                heads: int, hd: int, *, act_silu: bool = False,
                rot_dims: int = 0, positions=None, inv_freq=None,
-               cache=None, slot_mapping=None):
+               cache=None, slot_mapping=None, add_input: bool = False,
+               advance: bool = False, out=None):
     """Short causal convolution with carried inputs (see ref.short_conv).
     With `cache` [blocks, heads, block, hd] the result is scattered to the
-    tokens' slots and None is returned; else a new [T, heads*hd] tensor."""
+    tokens' slots and None is returned; else it goes to `out` (None: a new
+    [T, heads*hd] tensor). advance: the only reader of these channels of the
+    state, which moves past this step's rows as short_conv_state_ would do
+    it (x must cover every channel of the state)."""
     if x.is_cuda:
-        out = None
-        if cache is None:
+        if cache is None and out is None:
             out = torch.empty(x.shape[0], heads * hd, dtype=x.dtype,
                               device=x.device)
+        # decode rows: the convolution's threads own their channels and move
+        # the state themselves
+        fused = advance and cu_q is None
         _hyb().short_conv(out, cache, slot_mapping, x, w, bias, state,
                           state_off, slots, cu_q, ctx_lens, heads, hd,
-                          act_silu, rot_dims, positions, inv_freq)
+                          act_silu, rot_dims, positions, inv_freq, add_input,
+                          fused)
+        if advance and not fused:
+            short_conv_state_(state, x, slots, cu_q)
         return out
-    out = ref.short_conv(x, w, bias, state, state_off, slots, cu_q, ctx_lens,
-                         heads, hd, act_silu, rot_dims, positions, inv_freq)
+    y = ref.short_conv(x, w, bias, state, state_off, slots, cu_q, ctx_lens,
+                       heads, hd, act_silu, rot_dims, positions, inv_freq,
+                       add_input)
+    if advance:
+        short_conv_state_(state, x, slots, cu_q)
+    if out is not None:
+        out.copy_(y)
+    else:
+        out = y
     if cache is None:
         return out
     ref.store_paged(out, cache, slot_mapping)
@@ -282,10 +304,13 @@ def gated_group_norm(o, w, gate, eps: float, groups: int, *, act_silu: bool,
 def capped_attn(q, k_cache, v_cache, block_tables, cu_q, seq_lens,
                 heads: int, scale: float, cap: float, out, window: int = 0,
                 sink: Optional[torch.Tensor] = None, keep_first: int = 0,
-                head_scale: Optional[torch.Tensor] = None):
+                head_scale: Optional[torch.Tensor] = None,
+                chunked: bool = False):
     """out fp32 [T, heads, Dv] (written). cu_q None: decode rows. window > 0
     limits a query to the last `window` keys (itself included) and, with
-    keep_first, the first keep_first keys of the sequence; sink fp32 [heads]
+    keep_first, the first keep_first keys of the sequence; chunked: `window`
+    is the size of the chunks, counted from position 0, that the sequence
+    falls into, and a query sees its own chunk only. sink fp32 [heads]
     adds exp(sink_h) to the softmax denominator; head_scale fp32 [heads]
     multiplies the scores of a head."""
     if window <= 0:
@@ -293,11 +318,11 @@ def capped_attn(q, k_cache, v_cache, block_tables, cu_q, seq_lens,
     if q.is_cuda:
         _hyb().capped_attn(out, q, k_cache, v_cache, block_tables, cu_q,
                            seq_lens, heads, scale, cap, window, sink,
-                           keep_first, head_scale)
+                           keep_first, head_scale, chunked)
         return out
     out.copy_(ref.capped_attn(q, k_cache, v_cache, block_tables, cu_q,
                               seq_lens, heads, scale, cap, window, sink,
-                              keep_first, head_scale))
+                              keep_first, head_scale, chunked))
     return out
 
 
@@ -334,7 +359,9 @@ def rownorm_rope_store(q, k, v, q_w, k_w, eps: float, positions, inv_freq,
 def delta_rule(q, k, v, b, a, dt_bias, A_log, state, slots, cu_q, ctx_lens,
                groups: int, out, max_q_len: int = 0):
     """out fp32 [T, H, Dv] (written); see ref.delta_rule. q/k/v/b/a are row
-    views of the projections; state fp32 [slots, H, D, Dv] in place.
+    views of the projections; state fp32 [slots, H, D, Dv] in place. dt_bias
+    fp32 [H] with a [T, H]: one decay per head; fp32 [H*D] with a [T, H*D]:
+    one per head and key channel.
     max_q_len: host-known bound on the longest sequence chunk (0: unknown)."""
     if q.is_cuda:
         _hyb().delta_rule(out, q, k, v, b, a, dt_bias, A_log, state, slots,
@@ -358,21 +385,23 @@ def gelu_tanh_mul(x):
 # ---- rotary + unit head norm with paged store, PolyNorm, two-tensor gate ----
 def rope_headnorm_store(q, k, v, positions, inv_freq, rot_dims: int,
                         pairs: bool, unit_norm: bool, eps: float, heads: int,
-                        kv_heads: int, k_cache, v_cache, slot_mapping):
+                        kv_heads: int, k_cache, v_cache, slot_mapping,
+                        mscale: float = 1.0):
     """Rotary turn on the first rot_dims entries of every head of q [T,
     heads*D] and k [T, kv_heads*D] (`pairs`: entries 2i / 2i+1, else i / i +
-    rot_dims/2), then with unit_norm each head divided by its root mean
+    rot_dims/2; cos/sin scaled by mscale), then with unit_norm each head divided by its root mean
     square. Returns the new q as a contiguous tensor; k and v (None: the
     values are the keys) go into the paged caches at the tokens' slots."""
     if q.is_cuda:
         out = torch.empty(q.shape, dtype=q.dtype, device=q.device)
         _hyb().rope_headnorm_store(out, q, k, v, positions, inv_freq,
                                    rot_dims, pairs, unit_norm, eps, heads,
-                                   kv_heads, k_cache, v_cache, slot_mapping)
+                                   kv_heads, k_cache, v_cache, slot_mapping,
+                                   mscale)
         return out
     return ref.rope_headnorm_store(q, k, v, positions, inv_freq, rot_dims,
                                    pairs, unit_norm, eps, heads, kv_heads,
-                                   k_cache, v_cache, slot_mapping)
+                                   k_cache, v_cache, slot_mapping, mscale)
 
 
 def polynorm(z, coef, eps: float):
@@ -392,3 +421,44 @@ def gelu_tanh_gate(g, u):
         _hyb().gelu_tanh_gate(out, g, u)
         return out
     return ref.gelu_tanh_gate(g, u)
+
+
+# ---- depth average of the residual, clamped gate, expert GELU ---------------
+def depth_mix_norm(x_in, hist, level: int, m1, w1, m2, w2, m_scale: float, f,
+                   dwa, g1, g2, eps: float, out_dtype, x_out=None):
+    """One layer's result and what follows it in one pass over the row:
+    r = x_in + m_scale (m1' + m2') + f goes to hist[level] (fp32 [levels, T,
+    W]), x_out = sum_{j <= level} dwa[j] hist[j] (dwa None: r), and the next
+    sublayers' inputs x_out / rms(x_out) * g1 and * g2 (one number each) are
+    returned. m' = m / rms(m) * w with a weight w (fp32, vector or one
+    number), m without. x_in, m2, f, g2, x_out may be None."""
+    if m1.is_cuda:
+        h1 = torch.empty(m1.shape, dtype=out_dtype, device=m1.device)
+        h2 = None if g2 is None else torch.empty_like(h1)
+        _hyb().depth_mix_norm(h1, h2, x_out, x_in, hist, level, m1, w1, m2,
+                              w2, m_scale, f, dwa, g1, g2, eps)
+        return h1, h2
+    return ref.depth_mix_norm(x_in, hist, level, m1, w1, m2, w2, m_scale, f,
+                              dwa, g1, g2, eps, out_dtype, x_out)
+
+
+def clamped_glu(x, limit: float, alpha: float, shift: float):
+    """[..., 2F] -> g sigmoid(alpha g) (u + shift), g = min(first half,
+    limit), u = the second half clamped to +-limit."""
+    if x.is_cuda:
+        out = torch.empty(x.shape[:-1] + (x.shape[-1] // 2,), dtype=x.dtype,
+                          device=x.device)
+        _hyb().clamped_glu(out, x, limit, alpha, shift)
+        return out
+    return ref.clamped_glu(x, limit, alpha, shift)
+
+
+def gelu_scaled(x, scale=None, ids=None, wts=None):
+    """Exact GELU of s_r x[r] per row; s from `scale` (fp32 per row) or, for
+    rows in the order (expert, token), from a routing (ids, wts); see
+    ref.gelu_scaled."""
+    if x.is_cuda:
+        out = torch.empty_like(x)
+        _hyb().gelu_scaled(out, x, scale, ids, wts)
+        return out
+    return ref.gelu_scaled(x, scale, ids, wts)

@@ -200,10 +200,14 @@ def norm_sigmoid_gate(o, w, gate, eps, out_dtype, gate_cols=1):
     return (z * g).to(out_dtype)
 
 
-def rope_interleaved(x, positions, inv_freq, mscale, rot_dims):
+def rope_interleaved(x, positions, inv_freq, mscale, rot_dims, pairs=True):
     """Rotate pairs (2i, 2i+1) of the first rot_dims entries of the last
     dim of x [T, H, D] by angle pos * inv_freq[i]; cos/sin scaled by mscale.
-    Angles in fp64. Returns a new tensor."""
+    pairs False: entry i turns with entry i + rot_dims/2 instead. Angles in
+    fp64. Returns a new tensor."""
+    if not pairs:
+        return rope_halves(x, positions, inv_freq, rot_dims,
+                           mscale).to(x.dtype)
     a = positions.double()[:, None] * inv_freq.double()[None, :]
     cos = (torch.cos(a) * mscale).float()[:, None, :]
     sin = (torch.sin(a) * mscale).float()[:, None, :]
@@ -217,12 +221,12 @@ def rope_interleaved(x, positions, inv_freq, mscale, rot_dims):
 
 
 def latent_kv_store(dkv, norm_w, eps, positions, inv_freq, mscale, rot_dims,
-                    cache, slot_mapping, kv_rank):
+                    cache, slot_mapping, kv_rank, pairs=True):
     """cache row = [rmsnorm(dkv[:kv_rank]) * w | rope(dkv[kv_rank:])];
     cache [blocks, bs, kv_rank + rot]."""
     c = group_rmsnorm(dkv[:, :kv_rank], norm_w, eps, 1, torch.float32)
     kr = rope_interleaved(dkv[:, None, kv_rank:].float(), positions, inv_freq,
-                          mscale, rot_dims)[:, 0]
+                          mscale, rot_dims, pairs)[:, 0]
     row = torch.cat([c, kr], -1).to(cache.dtype)
     bs = cache.shape[1]
     flat = cache.view(-1, cache.shape[-1])
@@ -238,11 +242,13 @@ def _gather_latent(cache, table, L):
     return cache[idx].reshape(nblk * bs, -1)[:L].float()
 
 
-def latent_attn(q, cache, block_tables, cu_q, seq_lens, scale, kv_rank):
+def latent_attn(q, cache, block_tables, cu_q, seq_lens, scale, kv_rank,
+                window=0):
     """Causal softmax attention of per-head queries [T, H, W] against the
     shared latent rows [W] of the paged cache; values are the first kv_rank
     entries of each row. Sequence s has queries cu_q[s]:cu_q[s+1], the last
-    of which sits at position seq_lens[s]-1. Returns fp32 [T, H, kv_rank]."""
+    of which sits at position seq_lens[s]-1. window > 0: position i sees only
+    the keys j with i - j < window. Returns fp32 [T, H, kv_rank]."""
     T, H, W = q.shape
     out = torch.zeros(T, H, kv_rank, dtype=torch.float32, device=q.device)
     for s in range(len(seq_lens)):
@@ -251,7 +257,10 @@ def latent_attn(q, cache, block_tables, cu_q, seq_lens, scale, kv_rank):
         ctx = L - (q1 - q0)
         kv = _gather_latent(cache, block_tables[s], L)          # [L, W]
         sc = torch.einsum("thw,lw->thl", q[q0:q1].float(), kv) * scale
-        mask = torch.arange(L)[None, :] > (ctx + torch.arange(q1 - q0))[:, None]
+        qpos = (ctx + torch.arange(q1 - q0))[:, None]
+        mask = torch.arange(L)[None, :] > qpos
+        if window and window > 0:
+            mask = mask | (torch.arange(L)[None, :] <= qpos - window)
         sc = sc.masked_fill(mask[:, None, :], float("-inf"))
         p = torch.softmax(sc, -1)
         out[q0:q1] = torch.einsum("thl,lr->thr", p, kv[:, :kv_rank])
@@ -352,12 +361,13 @@ def _seq_ranges(T, slots, cu_q):
 
 
 def short_conv(x, w, bias, state, state_off, slots, cu_q, ctx_lens, heads, hd,
-               act_silu, rot_dims, positions, inv_freq):
+               act_silu, rot_dims, positions, inv_freq, add_input=False):
     """Causal per-channel convolution of x [T, C] (C = heads*hd) with w
     [C, taps]; earlier inputs of a sequence come from state[slot, i,
     state_off:state_off+C] (the input of position ctx - (taps-1) + i), zeros
     before position 0. Optional bias, SiLU, and an interleaved rotary turn of
-    the first rot_dims channels of every head. Returns [T, C] in x's dtype."""
+    the first rot_dims channels of every head; with add_input the result is
+    x plus all that. Returns [T, C] in x's dtype."""
     T, C = x.shape
     taps = w.shape[1]
     K1 = taps - 1
@@ -381,6 +391,8 @@ def short_conv(x, w, bias, state, state_off, slots, cu_q, ctx_lens, heads, hd,
     if rot_dims:
         out = rope_interleaved(out.view(T, heads, hd), positions, inv_freq,
                                1.0, rot_dims).reshape(T, C)
+    if add_input:
+        out = out + x.float()
     return out.to(x.dtype)
 
 
@@ -466,14 +478,16 @@ def store_paged(x, cache, slot_mapping):
 
 def capped_attn(q, k_cache, v_cache, block_tables, cu_q, seq_lens, heads,
                 scale, cap, window=0, sink=None, keep_first=0,
-                head_scale=None):
+                head_scale=None, chunked=False):
     """Causal softmax attention of q [T, heads*D] over the paged caches
     [blocks, n_kv, block, D|Dv]; scores scale * q.k, then cap * tanh(. /
     cap) when cap > 0. window > 0: position i sees only the keys j with
     i - j < window. sink [heads]: exp(sink_h) joins the softmax denominator
     (a key without a value). keep_first: with a window, the keys j <
-    keep_first stay visible as well. head_scale [heads]: one more score
-    multiplier per head. Returns fp32 [T, heads, Dv]."""
+    keep_first stay visible as well. chunked: the sequence falls into chunks
+    of `window` positions and i sees only the keys of its own chunk.
+    head_scale [heads]: one more score multiplier per head. Returns fp32
+    [T, heads, Dv]."""
     T = q.shape[0]
     nb, n_kv, bs, D = k_cache.shape
     Dv = v_cache.shape[3]
@@ -500,7 +514,9 @@ def capped_attn(q, k_cache, v_cache, block_tables, cu_q, seq_lens, heads,
         qpos = (ctx + torch.arange(q1 - q0))[:, None]
         mask = torch.arange(L)[None, :] > qpos
         if window and window > 0:
-            gone = torch.arange(L)[None, :] <= qpos - window
+            first = qpos // window * window if chunked \
+                else qpos - window + 1
+            gone = torch.arange(L)[None, :] < first
             if keep_first > 0:
                 gone = gone & (torch.arange(L)[None, :] >= keep_first)
             mask = mask | gone
@@ -531,14 +547,16 @@ def norm_residual_add(x, y, w1, eps, out_dtype, w_next=None):
             * w_next).to(out_dtype)
 
 
-def rope_halves(x, positions, inv_freq, rot_dims):
+def rope_halves(x, positions, inv_freq, rot_dims, mscale=1.0):
     """Entry i < rot_dims/2 of the last dim of x [T, H, D] turns together
-    with entry i + rot_dims/2 by pos * inv_freq[i] (fp64 angles)."""
+    with entry i + rot_dims/2 by pos * inv_freq[i] (fp64 angles); cos/sin
+    scaled by mscale."""
     if not rot_dims:
         return x.float()
     half = rot_dims // 2
     a = positions.double()[:, None] * inv_freq.double()[None, :]
-    cos, sin = torch.cos(a).float()[:, None, :], torch.sin(a).float()[:, None, :]
+    cos = (torch.cos(a) * mscale).float()[:, None, :]
+    sin = (torch.sin(a) * mscale).float()[:, None, :]
     xf = x.float()
     u, v = xf[..., :half], xf[..., half:rot_dims]
     return torch.cat([u * cos - v * sin, v * cos + u * sin,
@@ -568,7 +586,9 @@ def delta_rule(q, k, v, b, a, dt_bias, A_log, state, slots, cu_q, ctx_lens,
                groups):
     """Gated delta rule. Per head, with unit k and q (q also times
     D^-1/2), beta = sigmoid(b), g = exp(-exp(A_log) softplus(a + dt_bias)):
-    S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q. q/k
+    S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q. With dt_bias
+    [H*D] (and a [T, H*D]) there is one decay per key channel: g scales the
+    rows of S. q/k
     [T, groups*D] shared by the heads of a group; state fp32
     [slots, H, D, Dv]; returns fp32 [T, H, Dv]."""
     H, D, Dv = state.shape[1:]
@@ -582,8 +602,8 @@ def delta_rule(q, k, v, b, a, dt_bias, A_log, state, slots, cu_q, ctx_lens,
     qf, kf = unit(q) * D ** -0.5, unit(k)
     vf = v.float().view(T, H, Dv)
     beta = torch.sigmoid(b.float())
-    g = torch.exp(-torch.exp(A_log) * torch.nn.functional.softplus(
-        a.float() + dt_bias, threshold=30.0))
+    sp = torch.nn.functional.softplus(a.float() + dt_bias, threshold=30.0)
+    g = torch.exp(-torch.exp(A_log)[None, :, None] * sp.view(T, H, -1))
     out = torch.zeros(T, H, Dv, dtype=torch.float32)
     for s, t0, t1 in _seq_ranges(T, slots, cu_q):
         slot = int(slots[s])
@@ -592,7 +612,7 @@ def delta_rule(q, k, v, b, a, dt_bias, A_log, state, slots, cu_q, ctx_lens,
         else:
             S = torch.zeros(H, D, Dv, dtype=torch.float32)
         for t in range(t0, t1):
-            S = g[t][:, None, None] * S
+            S = g[t][:, :, None] * S
             u = beta[t][:, None] * (vf[t] - torch.einsum("hdv,hd->hv", S,
                                                          kf[t]))
             S = S + kf[t][:, :, None] * u[:, None, :]
@@ -613,20 +633,19 @@ def gelu_tanh_mul(x):
 # ---------------------------------------------------------------------------
 def rope_headnorm_store(q, k, v, positions, inv_freq, rot_dims, pairs,
                         unit_norm, eps, heads, kv_heads, k_cache, v_cache,
-                        slot_mapping):
+                        slot_mapping, mscale=1.0):
     """q [T, heads*D], k [T, kv_heads*D]: rotary turn on the first rot_dims
     entries of every head (`pairs`: entries 2i and 2i+1 turn together, else
-    i and i + rot_dims/2), then with `unit_norm` every head is divided by
-    its root mean square. Returns the new q; k and v (when given) go to the
+    i and i + rot_dims/2; cos/sin scaled by mscale), then with `unit_norm`
+    every head is divided by its root mean square. Returns the new q; k and v (when given) go to the
     paged caches."""
     T = q.shape[0]
 
     def prep(z, n):
         z = z.reshape(T, n, -1)
         if rot_dims:
-            z = (rope_interleaved(z.float(), positions, inv_freq, 1.0,
-                                  rot_dims) if pairs
-                 else rope_halves(z, positions, inv_freq, rot_dims))
+            z = rope_interleaved(z.float(), positions, inv_freq, mscale,
+                                 rot_dims, pairs)
         z = z.float()
         if unit_norm:
             z = z * torch.rsqrt(z.pow(2).mean(-1, keepdim=True) + eps)
@@ -652,3 +671,64 @@ def polynorm(z, coef, eps):
 def gelu_tanh_gate(g, u):
     """gelu_tanh(g) * u for two tensors of one shape, dtype of g."""
     return (F.gelu(g.float(), approximate="tanh") * u.float()).to(g.dtype)
+
+
+# ---------------------------------------------------------------------------
+# Depth average of the residual with two norms, clamped gate, expert GELU.
+# fp32 throughout.
+# ---------------------------------------------------------------------------
+def _unit_rms(x, eps):
+    return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+
+
+def depth_mix_norm(x_in, hist, level, m1, w1, m2, w2, m_scale, f, dwa, g1, g2,
+                   eps, out_dtype, x_out):
+    """r = x_in + m_scale (m1' + m2') + f, kept as hist[level]; x_out = sum_j
+    dwa[j] hist[j] over j <= level (dwa None: x_out = r); returns x_out /
+    rms(x_out) times g1 and times g2 (None: not formed). m' = m / rms(m) * w
+    with a weight (vector or one number), m without. x_in None: r starts at
+    zero."""
+    def part(m, w):
+        return m.float() if w is None else _unit_rms(m.float(), eps) * w
+    r = part(m1, w1)
+    if m2 is not None:
+        r = r + part(m2, w2)
+    r = r * m_scale
+    if f is not None:
+        r = r + f.float()
+    if x_in is not None:
+        r = r + x_in
+    hist[level] = r
+    x = r
+    if dwa is not None:
+        x = torch.einsum("j,jtw->tw", dwa, hist[:level + 1])
+    if x_out is not None:
+        x_out.copy_(x)
+    n = _unit_rms(x, eps)
+    return ((n * g1).to(out_dtype),
+            None if g2 is None else (n * g2).to(out_dtype))
+
+
+def clamped_glu(x, limit, alpha, shift):
+    """[..., 2F]: g = min(x[..., :F], limit), u = clamp(x[..., F:], -limit,
+    limit); g sigmoid(alpha g) (u + shift). dtype preserved."""
+    d = x.shape[-1] // 2
+    g = x[..., :d].float().clamp(max=limit)
+    u = x[..., d:].float().clamp(min=-limit, max=limit)
+    return (g * torch.sigmoid(alpha * g) * (u + shift)).to(x.dtype)
+
+
+def gelu_scaled(x, scale=None, ids=None, wts=None):
+    """Exact GELU of s_r * x[r] per row of x [..., F]. s: `scale` per row; or
+    rows in the order (expert, token) with the weight `wts` [T, top] of the
+    token's choice of that expert in `ids` [T, top] (rows of experts a token
+    did not choose are zero). dtype preserved."""
+    rows = x.numel() // x.shape[-1]
+    if ids is not None:
+        T = ids.shape[0]
+        s = torch.zeros(rows // T, T, dtype=torch.float32)
+        for k in range(ids.shape[1]):
+            s[ids[:, k].long(), torch.arange(T)] = wts[:, k]
+        scale = s.reshape(-1)
+    s = 1.0 if scale is None else scale.view(*x.shape[:-1], 1)
+    return F.gelu(x.float() * s).to(x.dtype)
