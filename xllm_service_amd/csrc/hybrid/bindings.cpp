@@ -29,7 +29,7 @@ template <typename T>
 void launch_rope_headnorm_store(T*, const T*, const T*, const T*, long, long,
                                 long, const long*, const double*, int, int,
                                 int, float, int, int, int, int, int, T*, T*,
-                                const long*, int, hipStream_t);
+                                const long*, int, float, hipStream_t);
 template <typename T>
 void launch_polynorm(T*, const T*, const float*, float, long, int, long,
                      hipStream_t);
@@ -49,25 +49,25 @@ void launch_rownorm_rope_store(T*, const T*, const T*, const T*, long, long,
 template <typename T>
 void launch_delta_rule(float*, const T*, const T*, const T*, const T*,
                        const T*, long, long, long, long, long, const float*,
-                       const float*, float*, const int*, const int*,
+                       const float*, int, float*, const int*, const int*,
                        const int*, int, int, int, int, int, int, int, float*,
                        hipStream_t);
 template <typename T>
 void launch_rope_interleaved(T*, const long*, const double*, float, int, int,
-                             int, long, long, int, hipStream_t);
+                             int, long, long, int, int, hipStream_t);
 template <typename T>
 void launch_latent_kv_store(T*, const T*, const float*, float, const long*,
                             const double*, float, int, const long*, int, int,
-                            int, long, hipStream_t);
+                            int, long, int, hipStream_t);
 template <typename T>
 void launch_latent_attn(float*, const T*, const T*, const int*, const int*,
                         const int*, int, int, int, int, int, int, int, float,
-                        long, hipStream_t);
+                        long, int, hipStream_t);
 int latent_attn_mfma_class(int W, int r);
 void launch_latent_attn_mfma(float*, float*, float*, const unsigned short*,
                              const unsigned short*, const int*, const int*,
                              const int*, int, int, int, int, int, int, int,
-                             float, int, hipStream_t);
+                             float, int, int, hipStream_t);
 template <typename T>
 void launch_decay_attn(float*, const T*, const T*, const T*, const float*,
                        float*, const int*, const int*, const int*, int, int,
@@ -95,9 +95,10 @@ template <typename T>
 void launch_softcap(float*, const T*, float, long, hipStream_t);
 template <typename T>
 void launch_short_conv(T*, long, T*, const long*, int, const T*, long,
-                       const T*, const T*, const T*, long, int, const int*,
+                       const T*, const T*, T*, long, int, const int*,
                        const int*, const int*, int, int, int, int, int, int,
-                       int, const long*, const double*, hipStream_t);
+                       int, const long*, const double*, int, int,
+                       hipStream_t);
 template <typename T>
 void launch_short_conv_state(T*, long, const T*, long, const int*, const int*,
                              int, int, int, hipStream_t);
@@ -116,13 +117,25 @@ void launch_capped_attn_mfma(float*, float*, float*, const unsigned short*,
                              const unsigned short*, const unsigned short*,
                              const int*, const int*, const int*, int, int, int,
                              int, int, int, int, int, float, float, long, int,
-                             int, const float*, int, const float*,
+                             int, const float*, int, const float*, int,
                              hipStream_t);
 template <typename T>
 void launch_capped_attn(float*, const T*, const T*, const T*, const int*,
                         const int*, const int*, int, int, int, int, int, int,
                         int, int, float, float, long, int, const float*, int,
-                        const float*, hipStream_t);
+                        const float*, int, hipStream_t);
+template <typename T, typename TF>
+void launch_depth_mix_norm(T*, T*, float*, const float*, float*, long, int,
+                           const T*, const float*, int, const T*,
+                           const float*, int, float, const TF*, const float*,
+                           const float*, const float*, float, int, int,
+                           hipStream_t);
+template <typename T>
+void launch_clamped_glu(T*, const T*, long, int, float, float, float,
+                        hipStream_t);
+template <typename T>
+void launch_gelu_scaled(T*, const T*, long, int, const float*, const int*,
+                        const float*, int, int, hipStream_t);
 }  // namespace hyb
 }  // namespace xllm
 
@@ -276,7 +289,7 @@ void rope_headnorm_store(Tensor q_out, Tensor q, Tensor k,
                          c10::optional<Tensor> v, Tensor pos, Tensor inv_freq,
                          long rot, bool pairs, bool unit, double eps,
                          long heads, long n_kv, Tensor k_cache,
-                         Tensor v_cache, Tensor slot_mapping) {
+                         Tensor v_cache, Tensor slot_mapping, double mscale) {
   CHK_ACT(q_out); CHK_ACT(q); CHK_ACT(k); CHK_I64C(pos);
   CHK_I64C(slot_mapping); CHK_ACT(k_cache); CHK_ACT(v_cache);
   TORCH_CHECK(q.dim() == 2 && k.dim() == 2 && q_out.is_contiguous() &&
@@ -307,9 +320,9 @@ void rope_headnorm_store(Tensor q_out, Tensor q, Tensor k,
     vs = v->stride(0);
   }
   if (is_f32(q))
-    hy::launch_rope_headnorm_store<float>(ptr<float>(q_out), ptr<float>(q), ptr<float>(k), (const float*)vp, q.stride(0), k.stride(0), vs, ptr<long>(pos), ptr<double>(inv_freq), rot, pairs, unit, eps, T, heads, n_kv, D, Dv, ptr<float>(k_cache), ptr<float>(v_cache), ptr<long>(slot_mapping), bs, cur());
+    hy::launch_rope_headnorm_store<float>(ptr<float>(q_out), ptr<float>(q), ptr<float>(k), (const float*)vp, q.stride(0), k.stride(0), vs, ptr<long>(pos), ptr<double>(inv_freq), rot, pairs, unit, eps, T, heads, n_kv, D, Dv, ptr<float>(k_cache), ptr<float>(v_cache), ptr<long>(slot_mapping), bs, mscale, cur());
   else
-    hy::launch_rope_headnorm_store<bf>(ptr<bf>(q_out), ptr<bf>(q), ptr<bf>(k), (const bf*)vp, q.stride(0), k.stride(0), vs, ptr<long>(pos), ptr<double>(inv_freq), rot, pairs, unit, eps, T, heads, n_kv, D, Dv, ptr<bf>(k_cache), ptr<bf>(v_cache), ptr<long>(slot_mapping), bs, cur());
+    hy::launch_rope_headnorm_store<bf>(ptr<bf>(q_out), ptr<bf>(q), ptr<bf>(k), (const bf*)vp, q.stride(0), k.stride(0), vs, ptr<long>(pos), ptr<double>(inv_freq), rot, pairs, unit, eps, T, heads, n_kv, D, Dv, ptr<bf>(k_cache), ptr<bf>(v_cache), ptr<long>(slot_mapping), bs, mscale, cur());
 }
 
 void gelu_tanh_mul(Tensor out, Tensor x) {
@@ -359,7 +372,8 @@ void rownorm_rope_store(Tensor q_out, Tensor q, Tensor k, Tensor v, Tensor wq,
 }
 
 // out fp32 [T, H, Dv]; state fp32 [slots, H, D, Dv]; q/k [T, groups*D],
-// v [T, H*Dv], b/a [T, H] row views (after convolution: q, k, v)
+// v [T, H*Dv], b [T, H] row views (after convolution: q, k, v); a [T, H] with
+// dt_bias [H], or a [T, H*D] with dt_bias [H*D] (one decay per key channel)
 void delta_rule(Tensor out, Tensor q, Tensor k, Tensor v, Tensor b, Tensor a,
                 Tensor dt_bias, Tensor A_log, Tensor state, Tensor slots,
                 c10::optional<Tensor> cu_q, Tensor ctx_lens, long groups,
@@ -375,12 +389,14 @@ void delta_rule(Tensor out, Tensor q, Tensor k, Tensor v, Tensor b, Tensor a,
   const int T = q.size(0);
   TORCH_CHECK(groups >= 1 && H % groups == 0 && q.size(1) == groups * D &&
               k.size(1) == groups * D && v.size(1) == H * Dv &&
-              b.size(1) == H && a.size(1) == H && k.size(0) == T &&
+              b.size(1) == H && k.size(0) == T &&
               v.size(0) == T && b.size(0) == T && a.size(0) == T &&
-              dt_bias.numel() == H && A_log.numel() == H,
+              (dt_bias.numel() == H || dt_bias.numel() == (long)H * D) &&
+              a.size(1) == dt_bias.numel() && A_log.numel() == H,
               "delta_rule: bad shapes");
   TORCH_CHECK(D <= 256, "key dim > 256 unsupported");
   TORCH_CHECK(out.numel() == (long)T * H * Dv);
+  const int ch = dt_bias.numel() != H;       // channel decays
   const int n_seqs = slots.numel();
   TORCH_CHECK(ctx_lens.numel() == n_seqs);
   const int* cu = nullptr;
@@ -416,9 +432,9 @@ void delta_rule(Tensor out, Tensor q, Tensor k, Tensor v, Tensor b, Tensor a,
   }
   float* wsp = max_chunks > 1 ? ptr<float>(ws) : nullptr;
   if (is_f32(q))
-    hy::launch_delta_rule<float>(ptr<float>(out), ptr<float>(q), ptr<float>(k), ptr<float>(v), ptr<float>(b), ptr<float>(a), q.stride(0), k.stride(0), v.stride(0), b.stride(0), a.stride(0), ptr<float>(dt_bias), ptr<float>(A_log), ptr<float>(state), ptr<int>(slots), cu, ptr<int>(ctx_lens), n_seqs, H, groups, D, Dv, chunk, max_chunks, wsp, cur());
+    hy::launch_delta_rule<float>(ptr<float>(out), ptr<float>(q), ptr<float>(k), ptr<float>(v), ptr<float>(b), ptr<float>(a), q.stride(0), k.stride(0), v.stride(0), b.stride(0), a.stride(0), ptr<float>(dt_bias), ptr<float>(A_log), ch, ptr<float>(state), ptr<int>(slots), cu, ptr<int>(ctx_lens), n_seqs, H, groups, D, Dv, chunk, max_chunks, wsp, cur());
   else
-    hy::launch_delta_rule<bf>(ptr<float>(out), ptr<bf>(q), ptr<bf>(k), ptr<bf>(v), ptr<bf>(b), ptr<bf>(a), q.stride(0), k.stride(0), v.stride(0), b.stride(0), a.stride(0), ptr<float>(dt_bias), ptr<float>(A_log), ptr<float>(state), ptr<int>(slots), cu, ptr<int>(ctx_lens), n_seqs, H, groups, D, Dv, chunk, max_chunks, wsp, cur());
+    hy::launch_delta_rule<bf>(ptr<float>(out), ptr<bf>(q), ptr<bf>(k), ptr<bf>(v), ptr<bf>(b), ptr<bf>(a), q.stride(0), k.stride(0), v.stride(0), b.stride(0), a.stride(0), ptr<float>(dt_bias), ptr<float>(A_log), ch, ptr<float>(state), ptr<int>(slots), cu, ptr<int>(ctx_lens), n_seqs, H, groups, D, Dv, chunk, max_chunks, wsp, cur());
 }
 
 void silu_mul(Tensor out, Tensor x) {
@@ -432,9 +448,10 @@ void silu_mul(Tensor out, Tensor x) {
   else hy::launch_silu_mul<bf>(ptr<bf>(out), ptr<bf>(x), rows, F, cur());
 }
 
-// x [T, H, D] view (unit inner stride); rotates x[..., off:off+rot_dims]
+// x [T, H, D] view (unit inner stride); rotates x[..., off:off+rot_dims],
+// entries 2i / 2i+1 (pairs) or i / i + rot_dims/2
 void rope_interleaved(Tensor x, Tensor pos, Tensor inv_freq, double mscale,
-                      long off, long rot_dims) {
+                      long off, long rot_dims, bool pairs) {
   CHK_ACT(x); CHK_I64C(pos);
   TORCH_CHECK(inv_freq.is_cuda() && inv_freq.dtype() == torch::kDouble &&
               inv_freq.is_contiguous());
@@ -443,15 +460,15 @@ void rope_interleaved(Tensor x, Tensor pos, Tensor inv_freq, double mscale,
               inv_freq.numel() == rot_dims / 2);
   const int T = x.size(0), H = x.size(1);
   if (is_f32(x))
-    hy::launch_rope_interleaved<float>(ptr<float>(x), ptr<long>(pos), ptr<double>(inv_freq), mscale, T, H, rot_dims / 2, x.stride(0), x.stride(1), off, cur());
+    hy::launch_rope_interleaved<float>(ptr<float>(x), ptr<long>(pos), ptr<double>(inv_freq), mscale, T, H, rot_dims / 2, x.stride(0), x.stride(1), off, !pairs, cur());
   else
-    hy::launch_rope_interleaved<bf>(ptr<bf>(x), ptr<long>(pos), ptr<double>(inv_freq), mscale, T, H, rot_dims / 2, x.stride(0), x.stride(1), off, cur());
+    hy::launch_rope_interleaved<bf>(ptr<bf>(x), ptr<long>(pos), ptr<double>(inv_freq), mscale, T, H, rot_dims / 2, x.stride(0), x.stride(1), off, !pairs, cur());
 }
 
 // cache [blocks, bs, r+rd]; dkv [T, r+rd] row view
 void latent_kv_store(Tensor cache, Tensor dkv, Tensor norm_w, double eps,
                      Tensor pos, Tensor inv_freq, double mscale,
-                     long rot_dims, Tensor slots, long kv_rank) {
+                     long rot_dims, Tensor slots, long kv_rank, bool pairs) {
   CHK_ACT(cache); CHK_ACT(dkv); CHK_F32C(norm_w); CHK_I64C(pos);
   CHK_I64C(slots);
   TORCH_CHECK(cache.is_contiguous() && cache.dim() == 3 && dkv.dim() == 2 &&
@@ -465,15 +482,15 @@ void latent_kv_store(Tensor cache, Tensor dkv, Tensor norm_w, double eps,
               inv_freq.numel() == rot_dims / 2 && pos.numel() == T &&
               slots.numel() == T);
   if (is_f32(dkv))
-    hy::launch_latent_kv_store<float>(ptr<float>(cache), ptr<float>(dkv), ptr<float>(norm_w), eps, ptr<long>(pos), ptr<double>(inv_freq), mscale, rot_dims, ptr<long>(slots), T, r, rd, dkv.stride(0), cur());
+    hy::launch_latent_kv_store<float>(ptr<float>(cache), ptr<float>(dkv), ptr<float>(norm_w), eps, ptr<long>(pos), ptr<double>(inv_freq), mscale, rot_dims, ptr<long>(slots), T, r, rd, dkv.stride(0), !pairs, cur());
   else
-    hy::launch_latent_kv_store<bf>(ptr<bf>(cache), ptr<bf>(dkv), ptr<float>(norm_w), eps, ptr<long>(pos), ptr<double>(inv_freq), mscale, rot_dims, ptr<long>(slots), T, r, rd, dkv.stride(0), cur());
+    hy::launch_latent_kv_store<bf>(ptr<bf>(cache), ptr<bf>(dkv), ptr<float>(norm_w), eps, ptr<long>(pos), ptr<double>(inv_freq), mscale, rot_dims, ptr<long>(slots), T, r, rd, dkv.stride(0), !pairs, cur());
 }
 
 // out fp32 [T, H, r]; q [T, H, r+rd] contiguous; cu_q None => decode
 void latent_attn(Tensor out, Tensor q, Tensor cache, Tensor block_tables,
                  c10::optional<Tensor> cu_q, Tensor seq_lens, double scale,
-                 long kv_rank) {
+                 long kv_rank, long window) {
   CHK_F32C(out); CHK_ACT(q); CHK_ACT(cache); CHK_I32C(block_tables);
   CHK_I32C(seq_lens);
   TORCH_CHECK(q.dim() == 3 && q.is_contiguous() && cache.is_contiguous() &&
@@ -484,6 +501,7 @@ void latent_attn(Tensor out, Tensor q, Tensor cache, Tensor block_tables,
   TORCH_CHECK(cache.size(2) == W && r > 0 && r <= W && r <= 64 * 16,
               "latent width mismatch or kv_rank > 1024");
   TORCH_CHECK(out.numel() == (long)T * H * r);
+  TORCH_CHECK(window >= 0 && window < (1L << 30), "bad window");
   const int n_seqs = seq_lens.numel();
   TORCH_CHECK(block_tables.size(0) == n_seqs);
   const int* cu = nullptr;
@@ -504,7 +522,9 @@ void latent_attn(Tensor out, Tensor q, Tensor cache, Tensor block_tables,
       // about one workgroup per CU measured best (batch 8/32/128 at 1k-4k
       // context): more parts only add fp32 partials to write and merge
       const int tps = (H + 63) / 64;
-      const long max_tiles = ((long)block_tables.size(1) * cache.size(1) + 31) / 32;
+      long max_tiles = ((long)block_tables.size(1) * cache.size(1) + 31) / 32;
+      if (window > 0)
+        max_tiles = std::min<long>(max_tiles, (window + 31) / 32 + 1);
       n_part = (int)std::min<long>(std::min<long>(32, (max_tiles + 1) / 2),
                                    std::max<long>(1, 256 / ((long)T * tps)));
       n_part = std::max(n_part, 1);
@@ -520,15 +540,16 @@ void latent_attn(Tensor out, Tensor q, Tensor cache, Tensor block_tables,
         ptr<float>(out), n_part > 1 ? ptr<float>(ws_acc) : nullptr,
         n_part > 1 ? ptr<float>(ws_ml) : nullptr, ptr<bf>(q), ptr<bf>(cache),
         ptr<int>(block_tables), cu, ptr<int>(seq_lens), T, n_seqs, H, r,
-        W - r, cache.size(1), block_tables.size(1), scale, n_part, cur());
+        W - r, cache.size(1), block_tables.size(1), scale, n_part, window,
+        cur());
     return;
   }
   const int nw = H < 4 ? H : 4;
   TORCH_CHECK((size_t)nw * W * 4 <= 64 * 1024, "query row too wide for LDS");
   if (is_f32(q))
-    hy::launch_latent_attn<float>(ptr<float>(out), ptr<float>(q), ptr<float>(cache), ptr<int>(block_tables), cu, ptr<int>(seq_lens), T, n_seqs, H, r, W - r, cache.size(1), block_tables.size(1), scale, q.stride(0), cur());
+    hy::launch_latent_attn<float>(ptr<float>(out), ptr<float>(q), ptr<float>(cache), ptr<int>(block_tables), cu, ptr<int>(seq_lens), T, n_seqs, H, r, W - r, cache.size(1), block_tables.size(1), scale, q.stride(0), window, cur());
   else
-    hy::launch_latent_attn<bf>(ptr<float>(out), ptr<bf>(q), ptr<bf>(cache), ptr<int>(block_tables), cu, ptr<int>(seq_lens), T, n_seqs, H, r, W - r, cache.size(1), block_tables.size(1), scale, q.stride(0), cur());
+    hy::launch_latent_attn<bf>(ptr<float>(out), ptr<bf>(q), ptr<bf>(cache), ptr<int>(block_tables), cu, ptr<int>(seq_lens), T, n_seqs, H, r, W - r, cache.size(1), block_tables.size(1), scale, q.stride(0), window, cur());
 }
 
 // out fp32 [T, H, Dv]; q,k [T, H*D] / v [T, H*Dv] row views (pre-activation)
@@ -601,17 +622,23 @@ void moe_route(Tensor ids, Tensor wts, Tensor z, long top, long n_groups,
                        normalize, cur());
 }
 
-// out fp32 [T, width]; y [R, width] contiguous; rows int32 [T, top] < R, a
+// out fp32 [T, width]; y [R, width] contiguous; rows int32 [T, top] < R; wts
+// fp32 [T, top] (absent: plain sum); a
 // negative row reads ident [T, width] (0 without one); extra [T, width] is
 // added
-void moe_combine(Tensor out, Tensor y, Tensor rows, Tensor wts,
+void moe_combine(Tensor out, Tensor y, Tensor rows, c10::optional<Tensor> wts,
                  c10::optional<Tensor> ident, c10::optional<Tensor> extra) {
-  CHK_F32C(out); CHK_ACT(y); CHK_I32C(rows); CHK_F32C(wts);
+  CHK_F32C(out); CHK_ACT(y); CHK_I32C(rows);
   TORCH_CHECK(y.is_contiguous() && out.dim() == 2 && rows.dim() == 2);
   const long T = out.size(0);
   const int width = out.size(1), top = rows.size(1);
-  TORCH_CHECK(rows.size(0) == T && wts.numel() == T * top &&
-              y.size(-1) == width);
+  TORCH_CHECK(rows.size(0) == T && y.size(-1) == width);
+  const float* wp = nullptr;
+  if (wts.has_value()) {
+    CHK_F32C(*wts);
+    TORCH_CHECK(wts->numel() == T * top);
+    wp = ptr<float>(*wts);
+  }
   const void *ip = nullptr, *ep = nullptr;
   long is = 0, es = 0;
   if (ident.has_value()) {
@@ -627,9 +654,9 @@ void moe_combine(Tensor out, Tensor y, Tensor rows, Tensor wts,
     ep = extra->data_ptr(); es = extra->stride(0);
   }
   if (is_f32(y))
-    hy::launch_moe_combine<float>(ptr<float>(out), ptr<float>(y), ptr<int>(rows), ptr<float>(wts), T, width, top, (const float*)ip, is, (const float*)ep, es, cur());
+    hy::launch_moe_combine<float>(ptr<float>(out), ptr<float>(y), ptr<int>(rows), wp, T, width, top, (const float*)ip, is, (const float*)ep, es, cur());
   else
-    hy::launch_moe_combine<bf>(ptr<float>(out), ptr<bf>(y), ptr<int>(rows), ptr<float>(wts), T, width, top, (const bf*)ip, is, (const bf*)ep, es, cur());
+    hy::launch_moe_combine<bf>(ptr<float>(out), ptr<bf>(y), ptr<int>(rows), wp, T, width, top, (const bf*)ip, is, (const bf*)ep, es, cur());
 }
 
 // x fp32 [T, S, W]; out [T, W] = layernorm(sum_s w_in[s] x[:, s]) * g + b
@@ -740,12 +767,15 @@ void softcap(Tensor out, Tensor x, double cap) {
 // filters w [heads*hd, taps]; the sequence's earlier inputs come from
 // state[slot, :, state_off : state_off + heads*hd]. Result to `out` (row
 // view) or into the paged `cache` [blocks, heads, block, hd] at slot_mapping.
+// add_input: x is added to the result. advance (decode rows, all channels of
+// the state): the state moves past this step's rows.
 void short_conv(c10::optional<Tensor> out, c10::optional<Tensor> cache,
                 c10::optional<Tensor> slot_mapping, Tensor x, Tensor w,
                 c10::optional<Tensor> bias, Tensor state, long state_off,
                 Tensor slots, c10::optional<Tensor> cu_q, Tensor ctx_lens,
                 long heads, long hd, bool act_silu, long rot_dims,
-                c10::optional<Tensor> pos, c10::optional<Tensor> inv_freq) {
+                c10::optional<Tensor> pos, c10::optional<Tensor> inv_freq,
+                bool add_input, bool advance) {
   CHK_ACT(x); CHK_ACT(w); CHK_ACT(state); CHK_I32C(slots); CHK_I32C(ctx_lens);
   TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && w.is_contiguous() &&
               state.dim() == 3 && state.is_contiguous() &&
@@ -754,6 +784,9 @@ void short_conv(c10::optional<Tensor> out, c10::optional<Tensor> cache,
   TORCH_CHECK(x.size(1) == C && w.size(0) == C && taps >= 1 && taps <= 16 &&
               state.size(1) == taps - 1 && state_off >= 0 &&
               state_off + C <= state.size(2), "short_conv: bad shapes");
+  TORCH_CHECK(!advance || (!cu_q.has_value() && state_off == 0 &&
+                           C == state.size(2)),
+              "short_conv: advance needs decode rows and the whole state");
   const int n_seqs = slots.numel();
   TORCH_CHECK(ctx_lens.numel() == n_seqs);
   const int* cu = nullptr;
@@ -808,9 +841,9 @@ void short_conv(c10::optional<Tensor> out, c10::optional<Tensor> cache,
     out_stride = out->stride(0);
   }
   if (is_f32(x))
-    hy::launch_short_conv<float>((float*)outp, out_stride, (float*)cachep, smp, bs, ptr<float>(x), x.stride(0), ptr<float>(w), (const float*)bp, ptr<float>(state), state.size(2), state_off, ptr<int>(slots), cu, ptr<int>(ctx_lens), T, n_seqs, heads, hd, taps, act_silu, rot_dims, posp, fp, cur());
+    hy::launch_short_conv<float>((float*)outp, out_stride, (float*)cachep, smp, bs, ptr<float>(x), x.stride(0), ptr<float>(w), (const float*)bp, ptr<float>(state), state.size(2), state_off, ptr<int>(slots), cu, ptr<int>(ctx_lens), T, n_seqs, heads, hd, taps, act_silu, rot_dims, posp, fp, add_input, advance, cur());
   else
-    hy::launch_short_conv<bf>((bf*)outp, out_stride, (bf*)cachep, smp, bs, ptr<bf>(x), x.stride(0), ptr<bf>(w), (const bf*)bp, ptr<bf>(state), state.size(2), state_off, ptr<int>(slots), cu, ptr<int>(ctx_lens), T, n_seqs, heads, hd, taps, act_silu, rot_dims, posp, fp, cur());
+    hy::launch_short_conv<bf>((bf*)outp, out_stride, (bf*)cachep, smp, bs, ptr<bf>(x), x.stride(0), ptr<bf>(w), (const bf*)bp, ptr<bf>(state), state.size(2), state_off, ptr<int>(slots), cu, ptr<int>(ctx_lens), T, n_seqs, heads, hd, taps, act_silu, rot_dims, posp, fp, add_input, advance, cur());
 }
 
 // state [slots, taps-1, C] <- the last taps-1 inputs after this step's rows
@@ -935,7 +968,7 @@ void capped_attn(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
                  Tensor block_tables, c10::optional<Tensor> cu_q,
                  Tensor seq_lens, long heads, double scale, double cap,
                  long window, c10::optional<Tensor> sink, long keep_first,
-                 c10::optional<Tensor> head_scale) {
+                 c10::optional<Tensor> head_scale, bool chunked) {
   CHK_F32C(out); CHK_ACT(q); CHK_ACT(k_cache); CHK_ACT(v_cache);
   CHK_I32C(block_tables); CHK_I32C(seq_lens);
   TORCH_CHECK(q.dim() == 2 && k_cache.dim() == 4 && v_cache.dim() == 4 &&
@@ -1008,14 +1041,120 @@ void capped_attn(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
         n_part > 1 ? ptr<float>(ws_ml) : nullptr, ptr<bf>(q), ptr<bf>(k_cache),
         ptr<bf>(v_cache), ptr<int>(block_tables), cu, ptr<int>(seq_lens), T,
         n_seqs, heads, n_kv, D, Dv, bs, block_tables.size(1), scale, cap,
-        q.stride(0), n_part, window, sinkp, keep_first, hsp, cur());
+        q.stride(0), n_part, window, sinkp, keep_first, hsp, chunked, cur());
     return;
   }
   TORCH_CHECK((size_t)4 * D * 4 <= 64 * 1024, "query row too wide for LDS");
   if (is_f32(q))
-    hy::launch_capped_attn<float>(ptr<float>(out), ptr<float>(q), ptr<float>(k_cache), ptr<float>(v_cache), ptr<int>(block_tables), cu, ptr<int>(seq_lens), T, n_seqs, heads, n_kv, D, Dv, bs, block_tables.size(1), scale, cap, q.stride(0), window, sinkp, keep_first, hsp, cur());
+    hy::launch_capped_attn<float>(ptr<float>(out), ptr<float>(q), ptr<float>(k_cache), ptr<float>(v_cache), ptr<int>(block_tables), cu, ptr<int>(seq_lens), T, n_seqs, heads, n_kv, D, Dv, bs, block_tables.size(1), scale, cap, q.stride(0), window, sinkp, keep_first, hsp, chunked, cur());
   else
-    hy::launch_capped_attn<bf>(ptr<float>(out), ptr<bf>(q), ptr<bf>(k_cache), ptr<bf>(v_cache), ptr<int>(block_tables), cu, ptr<int>(seq_lens), T, n_seqs, heads, n_kv, D, Dv, bs, block_tables.size(1), scale, cap, q.stride(0), window, sinkp, keep_first, hsp, cur());
+    hy::launch_capped_attn<bf>(ptr<float>(out), ptr<bf>(q), ptr<bf>(k_cache), ptr<bf>(v_cache), ptr<int>(block_tables), cu, ptr<int>(seq_lens), T, n_seqs, heads, n_kv, D, Dv, bs, block_tables.size(1), scale, cap, q.stride(0), window, sinkp, keep_first, hsp, chunked, cur());
+}
+
+// One layer's result and what follows it, see depth_mix.hip. h1 (h2) [T, W]
+// contiguous; m1, m2 of h1's type; f of that type or fp32; hist fp32
+// [levels, T, W]; w1, w2 fp32 with W or 1 entries; dwa fp32 with level + 1
+// entries; g1, g2 one entry each
+void depth_mix_norm(Tensor h1, c10::optional<Tensor> h2,
+                    c10::optional<Tensor> x_out, c10::optional<Tensor> x_in,
+                    Tensor hist, long level, Tensor m1,
+                    c10::optional<Tensor> w1, c10::optional<Tensor> m2,
+                    c10::optional<Tensor> w2, double m_scale,
+                    c10::optional<Tensor> f, c10::optional<Tensor> dwa,
+                    Tensor g1, c10::optional<Tensor> g2, double eps) {
+  CHK_ACT(h1); CHK_F32C(hist); CHK_ACT(m1); CHK_F32C(g1);
+  TORCH_CHECK(h1.dim() == 2 && h1.is_contiguous() && hist.dim() == 3);
+  const int T = h1.size(0), W = h1.size(1);
+  TORCH_CHECK(hist.size(1) == T && hist.size(2) == W && level >= 0 &&
+              level < hist.size(0) && g1.numel() == 1,
+              "depth_mix_norm: bad shapes");
+  TORCH_CHECK((size_t)W * 4 <= 60 * 1024, "width too large for LDS");
+  auto act = [&](const Tensor& t) -> const void* {      // [T, W] of h1's type
+    TORCH_CHECK(t.is_cuda() && t.is_contiguous() && t.dim() == 2 &&
+                t.size(0) == T && t.size(1) == W && t.dtype() == h1.dtype(),
+                "depth_mix_norm: bad sublayer output");
+    return t.data_ptr();
+  };
+  auto f32 = [&](const c10::optional<Tensor>& t, long n) -> float* {
+    if (!t.has_value()) return nullptr;
+    CHK_F32C(*t);
+    TORCH_CHECK(n < 0 ? (t->numel() == 1 || t->numel() == W)
+                      : t->numel() == n, "depth_mix_norm: bad fp32 operand");
+    return ptr<float>(*t);
+  };
+  const void* m1p = act(m1);
+  const void* m2p = m2.has_value() ? act(*m2) : nullptr;
+  const void* h2p = h2.has_value() ? act(*h2) : nullptr;
+  TORCH_CHECK(!h2.has_value() || g2.has_value());
+  const long n = (long)T * W;
+  const float* w1p = f32(w1, -1);
+  const float* w2p = f32(w2, -1);
+  const int w1n = w1p ? w1->numel() : 0, w2n = w2p ? w2->numel() : 0;
+  float* xo = f32(x_out, n);
+  const float* xi = f32(x_in, n);
+  const float* dp = f32(dwa, level + 1);
+  const float* g2p = f32(g2, 1);
+  const void* fp = nullptr;
+  bool f_f32 = is_f32(h1);
+  if (f.has_value()) {
+    CHK_ACT(*f);
+    TORCH_CHECK(f->is_contiguous() && f->numel() == n &&
+                (is_f32(*f) || f->dtype() == h1.dtype()));
+    fp = f->data_ptr();
+    f_f32 = is_f32(*f);
+  }
+#define DM_CALL(T_, TF_)                                                      \
+  hy::launch_depth_mix_norm<T_, TF_>(                                         \
+      ptr<T_>(h1), (T_*)h2p, xo, xi, ptr<float>(hist), n, level,              \
+      (const T_*)m1p, w1p, w1n, (const T_*)m2p, w2p, w2n, m_scale,            \
+      (const TF_*)fp, dp, ptr<float>(g1), g2p, eps, T, W, cur())
+  if (is_f32(h1)) DM_CALL(float, float);
+  else if (f_f32) DM_CALL(bf, float);
+  else DM_CALL(bf, bf);
+#undef DM_CALL
+}
+
+void clamped_glu(Tensor out, Tensor x, double limit, double alpha,
+                 double shift) {
+  CHK_ACT(out); CHK_ACT(x);
+  TORCH_CHECK(out.is_contiguous() && x.is_contiguous() &&
+              out.dtype() == x.dtype());
+  const int F = out.size(-1);
+  TORCH_CHECK(x.size(-1) == 2 * F && x.numel() == 2 * out.numel());
+  const long rows = F ? out.numel() / F : 0;
+  if (is_f32(x)) hy::launch_clamped_glu<float>(ptr<float>(out), ptr<float>(x), rows, F, limit, alpha, shift, cur());
+  else hy::launch_clamped_glu<bf>(ptr<bf>(out), ptr<bf>(x), rows, F, limit, alpha, shift, cur());
+}
+
+// out like x [..., F]; scale fp32 one per row, or ids int32 / wts fp32
+// [T, top] for rows in the order (expert, token)
+void gelu_scaled(Tensor out, Tensor x, c10::optional<Tensor> scale,
+                 c10::optional<Tensor> ids, c10::optional<Tensor> wts) {
+  CHK_ACT(out); CHK_ACT(x);
+  TORCH_CHECK(out.is_contiguous() && x.is_contiguous() &&
+              out.dtype() == x.dtype() && out.numel() == x.numel());
+  const int F = x.size(-1);
+  const long rows = F ? x.numel() / F : 0;
+  const float *sp = nullptr, *wp = nullptr;
+  const int* ip = nullptr;
+  int tokens = 1, top = 0;
+  if (scale.has_value()) {
+    CHK_F32C(*scale);
+    TORCH_CHECK(scale->numel() == rows && !ids.has_value());
+    sp = ptr<float>(*scale);
+  }
+  if (ids.has_value()) {
+    TORCH_CHECK(wts.has_value());
+    CHK_I32C(*ids); CHK_F32C(*wts);
+    TORCH_CHECK(ids->dim() == 2 && ids->size(0) > 0 &&
+                rows % ids->size(0) == 0 && wts->numel() == ids->numel());
+    ip = ptr<int>(*ids);
+    wp = ptr<float>(*wts);
+    tokens = ids->size(0);
+    top = ids->size(1);
+  }
+  if (is_f32(x)) hy::launch_gelu_scaled<float>(ptr<float>(out), ptr<float>(x), rows, F, sp, ip, wp, tokens, top, cur());
+  else hy::launch_gelu_scaled<bf>(ptr<bf>(out), ptr<bf>(x), rows, F, sp, ip, wp, tokens, top, cur());
 }
 
 }  // namespace
@@ -1048,4 +1187,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("rope_headnorm_store", &rope_headnorm_store);
   m.def("polynorm", &polynorm);
   m.def("gelu_tanh_gate", &gelu_tanh_gate);
+  m.def("depth_mix_norm", &depth_mix_norm);
+  m.def("clamped_glu", &clamped_glu);
+  m.def("gelu_scaled", &gelu_scaled);
 }

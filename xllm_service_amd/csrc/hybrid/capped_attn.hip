@@ -6,7 +6,8 @@
 //   o_i  = sum_j softmax_j(s_ij) v_j        over keys j <= i
 //
 // Optional: a sliding window (only the keys with i - j < window are seen; with
-// keep_first the keys j < keep_first stay visible beside it), a per-head sink,
+// keep_first the keys j < keep_first stay visible beside it) or chunks (only
+// the keys with the same floor(. / window) are seen), a per-head sink,
 // a score without key or value whose exponential joins the softmax
 // denominator, and one more score multiplier per head.
 //
@@ -32,7 +33,7 @@ __global__ void capped_attn_kernel(
     const int* __restrict__ seq_lens, int n_seqs, int heads, int n_kv, int D,
     int Dv, int block_size, int table_width, float scale, float cap,
     long q_row_stride, int window, const float* __restrict__ sink,
-    int keep_first, const float* __restrict__ head_scale) {
+    int keep_first, const float* __restrict__ head_scale, int chunked) {
   extern __shared__ float smem[];
   const int t = blockIdx.x;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
@@ -73,7 +74,8 @@ __global__ void capped_attn_kernel(
 
   // two key ranges: the kept first keys that lie before the window, then
   // the window itself (all keys without one)
-  const int k_first = window > 0 ? max(0, n_keys - window) : 0;
+  const int k_first = window <= 0 ? 0
+      : chunked ? (n_keys - 1) / window * window : max(0, n_keys - window);
   const int kept = window > 0 ? min(keep_first, k_first) : 0;
   for (int seg = 0; seg < 2; ++seg) {
   const int seg_lo = seg == 0 ? 0 : k_first;
@@ -137,7 +139,8 @@ void launch_capped_attn(float* out, const T* q, const T* k_cache,
                         int block_size, int table_width, float scale,
                         float cap, long q_row_stride, int window,
                         const float* sink, int keep_first,
-                        const float* head_scale, hipStream_t st) {
+                        const float* head_scale, int chunked,
+                        hipStream_t st) {
   if (tokens == 0) return;
   const int nw = heads < 4 ? heads : 4;
   dim3 grid(tokens, (heads + nw - 1) / nw);
@@ -145,14 +148,15 @@ void launch_capped_attn(float* out, const T* q, const T* k_cache,
                      (size_t)nw * D * sizeof(float), st, out, q, k_cache,
                      v_cache, block_tables, cu_q, seq_lens, n_seqs, heads,
                      n_kv, D, Dv, block_size, table_width, scale, cap,
-                     q_row_stride, window, sink, keep_first, head_scale);
+                     q_row_stride, window, sink, keep_first, head_scale,
+                     chunked);
 }
 
 #define INST_CA(T)                                                          \
   template void launch_capped_attn<T>(                                      \
       float*, const T*, const T*, const T*, const int*, const int*,         \
       const int*, int, int, int, int, int, int, int, int, float, float,     \
-      long, int, const float*, int, const float*, hipStream_t);
+      long, int, const float*, int, const float*, int, hipStream_t);
 INST_CA(float)
 INST_CA(unsigned short)
 

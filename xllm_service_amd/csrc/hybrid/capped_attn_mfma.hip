@@ -41,7 +41,9 @@
 // keep_first, the keys [0, keep_first) as well; the tile loop runs over the
 // leading tiles that hold kept keys and then from the first tile any row of
 // the workgroup needs (one list of tiles, split evenly over the context
-// partitions). Sink: exp(sink_h) joins the denominator once, at the end (or
+// partitions). Chunks: `window` is the chunk size and a row sees the keys of
+// its own chunk up to itself; the rows of a workgroup may lie in several
+// chunks. Sink: exp(sink_h) joins the denominator once, at the end (or
 // in the merge kernel). head_scale: one more score multiplier per head.
 //
 // Fragment layouts of __builtin_amdgcn_mfma_f32_16x16x32_bf16 (lane l):
@@ -86,7 +88,7 @@ capped_attn_mfma_kernel(
     const int* __restrict__ seq_lens, int n_seqs, int heads, int n_kv, int D,
     int Dv, int block_size, int table_width, float scale, float cap,
     long q_stride, int n_part, int window, const float* __restrict__ sink,
-    int keep_first, const float* __restrict__ head_scale) {
+    int keep_first, const float* __restrict__ head_scale, int chunked) {
   extern __shared__ unsigned short cm_lds[];      // [key image | value image]
   __shared__ int tbl[512];                        // block ids of this key range
   constexpr int RT = 4 / CS;                      // row tiles per workgroup
@@ -131,7 +133,11 @@ capped_attn_mfma_kernel(
   const int kmax = ctx + last_row / per + 1;         // keys any row here sees
   const int n_tiles = (kmax + CM_KT - 1) / CM_KT;
   // first key the earliest row of this workgroup sees
-  const int kmin = window > 0 ? max(0, ctx + row0 / per + 1 - window) : 0;
+  auto first_key = [&](int lim) {    // of a row that sees keys below lim
+    return window <= 0 ? 0
+        : chunked ? (lim - 1) / window * window : max(0, lim - window);
+  };
+  const int kmin = first_key(ctx + row0 / per + 1);
   const int t_first = kmin / CM_KT;
   // tile list: [0, t_keep) then [t_first, n_tiles)
   const int t_keep = (window > 0 && keep_first > 0)
@@ -151,7 +157,7 @@ capped_attn_mfma_kernel(
   const bool wave_on = row0 + rt * 16 < rows_in_seq;
   const bool row_ok = rho < rows_in_seq;
   const int limit = row_ok ? ctx + rho / per + 1 : 0;
-  const int lo = window > 0 ? max(0, limit - window) : 0;
+  const int lo = row_ok ? first_key(limit) : 0;
   const int head = kvh * per + (row_ok ? rho % per : 0);
   const long tok = q0 + (row_ok ? rho / per : 0);
   const long grow = tok * heads + head;              // row in [T*H]
@@ -409,7 +415,8 @@ void launch_capped_attn_mfma(float* out, float* ws_acc, float* ws_ml,
                              int block_size, int table_width, float scale,
                              float cap, long q_stride, int n_part, int window,
                              const float* sink, int keep_first,
-                             const float* head_scale, hipStream_t st) {
+                             const float* head_scale, int chunked,
+                             hipStream_t st) {
   if (tokens == 0) return;
   const int cls = capped_attn_mfma_class(D, Dv);
   const int per = heads / n_kv;
@@ -428,7 +435,7 @@ void launch_capped_attn_mfma(float* out, float* ws_acc, float* ws_ml,
                      q, k_cache, v_cache, block_tables, cu_q, seq_lens,      \
                      n_seqs, heads, n_kv, D, Dv, block_size, table_width,    \
                      scale, cap, q_stride, n_part, window, sink, keep_first, \
-                     head_scale)
+                     head_scale, chunked)
 #define CM_BY_CS(KQ, NO)                                                     \
   do {                                                                       \
     if (cs == 4) CM_LAUNCH(KQ, NO, 4);                                       \

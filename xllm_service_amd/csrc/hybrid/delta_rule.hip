@@ -5,12 +5,17 @@
 //
 // with k_t, q_t made unit vectors per head (x / sqrt(sum x^2 + 1e-6)), q_t
 // also times D^-1/2, beta_t = sigmoid(b_t), g_t = exp(-exp(A_log_h)
-// softplus(a_t + dt_bias_h)). q and k are shared by the heads of a group.
-// Everything below is fp32; only the loads convert.
+// softplus(a_t + dt_bias_h)) per head, or per head and key channel (a_t and
+// dt_bias then have H*D entries and g_t scales the rows of S). q and k are
+// shared by the heads of a group. Everything below is fp32; only the loads
+// convert.
 //
 // With a = S_old^T k and c = S_old^T q the step is one pass of reductions
 // and one pass of updates over the state a thread holds in registers:
 //   u = beta (v - g a);  o = g c + (k . q) u;  S = g S_old + k u^T
+// With channel decays (CH) the first pass scales the rows on the way and a, c
+// are those of the scaled state:
+//   S = g S_old;  u = beta (v - S^T k);  o = S^T q + (k . q) u;  S += k u^T
 // The unit scales are folded into the reduced sums (a, c) and into u, so the
 // staged rows stay as loaded.
 //
@@ -25,7 +30,7 @@
 // float4 row pieces and sums the row groups' partials through LDS.
 //
 // Long chunks run piece-parallel. A token maps the state linearly,
-//   S <- g (I - beta k k^T) S + beta k v^T,
+//   S <- (I - beta k k^T) diag(g) S + beta k v^T,
 // so a piece of tokens maps S to M S + N with M [D, D] the product of its
 // token matrices and N [D, Dv] what the piece builds from a zero state. M is
 // what the same recurrence makes of an identity state with zero values:
@@ -71,13 +76,19 @@ struct DRArgs {
   int heads, groups, D, Dv;
 };
 
-// decay and write strength of token `row`, head h
+// decay of token `row`: entry e of the a row, A_log of head h
 template <typename T>
+XLLM_DEV float dr_decay(const DRArgs<T>& A, long row, int h, int e) {
+  const float dt = dr_softplus(IO<T>::ld(A.a + row * A.a_stride + e) +
+                               A.dt_bias[e]);
+  return expf(-expf(A.A_log[h]) * dt);
+}
+
+// decay (1 with channel decays) and write strength of token `row`, head h
+template <typename T, bool CH>
 XLLM_DEV void dr_gates(const DRArgs<T>& A, long row, int h, float* g,
                        float* beta) {
-  const float dt = dr_softplus(IO<T>::ld(A.a + row * A.a_stride + h) +
-                               A.dt_bias[h]);
-  *g = expf(-expf(A.A_log[h]) * dt);
+  *g = CH ? 1.0f : dr_decay<T>(A, row, h, h);
   *beta = 1.0f / (1.0f + expf(-IO<T>::ld(A.b + row * A.b_stride + h)));
 }
 
@@ -88,7 +99,8 @@ XLLM_DEV void dr_gates(const DRArgs<T>& A, long row, int h, float* g,
 // mode 2: the same tokens from the state the scan left in the record's first
 //         Dv columns; outputs written, nothing stored
 // NOOUT: a launch of mode 1 only; the read-out sums are not formed at all.
-template <typename T, int CPT, bool NOOUT>
+// CH: one decay per key channel.
+template <typename T, int CPT, bool NOOUT, bool CH>
 __global__ void __launch_bounds__(256) delta_rule_kernel(
     float* __restrict__ out, DRArgs<T> A, float* __restrict__ state,
     const int* __restrict__ slots, const int* __restrict__ cu_q,
@@ -101,6 +113,7 @@ __global__ void __launch_bounds__(256) delta_rule_kernel(
   float* ks = qs + DR_TC * D;             // [TC][D]
   float* vs = ks + DR_TC * D;             // [TC][VS]
   float* sc = vs + DR_TC * VS;            // [TC][NS]
+  float* gs = sc + DR_TC * DR_NS;         // [TC][D] (CH)
 
   const int s = blockIdx.x / max_chunks, cidx = blockIdx.x % max_chunks;
   const int h = blockIdx.y, v0 = blockIdx.z * VS;
@@ -170,6 +183,7 @@ __global__ void __launch_bounds__(256) delta_rule_kernel(
       const long row = tb + tt;
       qs[idx] = IO<T>::ld(A.q + row * A.q_stride + kg * D + i);
       ks[idx] = IO<T>::ld(A.k + row * A.k_stride + kg * D + i);
+      if (CH) gs[idx] = dr_decay<T>(A, row, h, h * D + i);
     }
     for (int idx = tid; idx < nt * VS; idx += 256) {
       const int tt = idx / VS, jj = idx - tt * VS;
@@ -178,7 +192,8 @@ __global__ void __launch_bounds__(256) delta_rule_kernel(
           ? IO<T>::ld(A.v + row * A.v_stride + h * Dv + v0 + jj) : 0.f;
     }
     if (tid < nt)
-      dr_gates<T>(A, tb + tid, h, sc + tid * DR_NS + 3, sc + tid * DR_NS + 4);
+      dr_gates<T, CH>(A, tb + tid, h, sc + tid * DR_NS + 3,
+                      sc + tid * DR_NS + 4);
     __syncthreads();
     {                                     // unit scales: 16 lanes per token
       const int tt = tid / DR_R;          // DR_TC * DR_R == 256 threads
@@ -210,8 +225,10 @@ __global__ void __launch_bounds__(256) delta_rule_kernel(
         const int i = r + DR_R * m;
         if (m < M && i < D) {
           const float kk = ks[tt * D + i], qq = qs[tt * D + i];
+          const float gg = CH ? gs[tt * D + i] : 1.f;
 #pragma unroll
           for (int c = 0; c < CPT; ++c) {
+            if (CH) S[m][c] *= gg;
             ak[c] += S[m][c] * kk;
             if (!NOOUT) aq[c] += S[m][c] * qq;
           }
@@ -232,7 +249,8 @@ __global__ void __launch_bounds__(256) delta_rule_kernel(
         if (m < M && i < D) {
           const float kk = ks[tt * D + i];
 #pragma unroll
-          for (int c = 0; c < CPT; ++c) S[m][c] = g * S[m][c] + kk * uk[c];
+          for (int c = 0; c < CPT; ++c)
+            S[m][c] = (CH ? S[m][c] : g * S[m][c]) + kk * uk[c];
         }
       }
       if (!NOOUT && mode != 1 && r == 0) {
@@ -390,7 +408,7 @@ __global__ void __launch_bounds__(64 * KB) delta_rule_scan_kernel(
 // rows rg, rg+RG, ... (NR of them, float4 each, kept in registers between the
 // reduction pass and the update pass); the RG row groups' partial sums meet
 // in LDS.
-template <typename T, int NR>
+template <typename T, int NR, bool CH>
 __global__ void __launch_bounds__(256) delta_rule_decode_kernel(
     float* __restrict__ out, DRArgs<T> A, float* __restrict__ state,
     const int* __restrict__ slots, const int* __restrict__ ctx_lens) {
@@ -406,12 +424,14 @@ __global__ void __launch_bounds__(256) delta_rule_decode_kernel(
   const int kg = h / (heads / A.groups);
   const int TCn = Dv >> 2, RG = 256 / TCn;
   float* pq = pa + RG * Dv;         // [RG][Dv] partial S^T q
+  float* gs = pq + RG * Dv;         // [D] channel decays (CH)
   const int rg = tid / TCn, tc = tid - rg * TCn;
   float sq = 0.f, sk = 0.f, skq = 0.f;
   for (int i = tid; i < D; i += 256) {
     const float qv = IO<T>::ld(A.q + s * A.q_stride + kg * D + i);
     const float kv = IO<T>::ld(A.k + s * A.k_stride + kg * D + i);
     qs[i] = qv; ks[i] = kv;
+    if (CH) gs[i] = dr_decay<T>(A, s, h, h * D + i);
     sq += qv * qv; sk += kv * kv; skq += qv * kv;
   }
   for (int i = tid; i < Dv; i += 256)
@@ -430,7 +450,7 @@ __global__ void __launch_bounds__(256) delta_rule_decode_kernel(
   const float qscale = 1.0f / sqrtf((float)D) / sqrtf(sq + 1e-6f);
   const float kq = skq * kscale * qscale;
   float g, beta;
-  dr_gates<T>(A, s, h, &g, &beta);
+  dr_gates<T, CH>(A, s, h, &g, &beta);
   const int slot = slots[s];
   const bool load = slot >= 0 && ctx_lens[s] > 0;
   float* sp = state + (((long)max(slot, 0) * heads + h) * D) * (long)Dv + 4 * tc;
@@ -443,6 +463,10 @@ __global__ void __launch_bounds__(256) delta_rule_decode_kernel(
       S[n] = make_float4(0.f, 0.f, 0.f, 0.f);
       if (i < D) {
         if (load) S[n] = *reinterpret_cast<const float4*>(sp + (long)i * Dv);
+        if (CH) {
+          const float gi = gs[i];
+          S[n].x *= gi; S[n].y *= gi; S[n].z *= gi; S[n].w *= gi;
+        }
         const float ki = ks[i], qi = qs[i];
         ak.x += S[n].x * ki; ak.y += S[n].y * ki;
         ak.z += S[n].z * ki; ak.w += S[n].w * ki;
@@ -483,24 +507,24 @@ __global__ void __launch_bounds__(256) delta_rule_decode_kernel(
   }
 }
 
-template <typename T, int CPT>
+template <typename T, int CPT, bool CH>
 void launch_delta_rule_cpt(float* out, const DRArgs<T>& A, float* state,
                            const int* slots, const int* cu_q,
                            const int* ctx_lens, int n_seqs, int chunk,
                            int max_chunks, float* ws, hipStream_t st) {
   constexpr int VS = DR_CG * CPT;
   const int D = A.D, Dv = A.Dv;
-  const size_t lds = (size_t)(2 * DR_TC * D + DR_TC * VS + DR_TC * DR_NS) *
-                     sizeof(float);
+  const size_t lds = (size_t)((CH ? 3 : 2) * DR_TC * D + DR_TC * VS +
+                              DR_TC * DR_NS) * sizeof(float);
   const int vz = (Dv + VS - 1) / VS;
   if (ws == nullptr || max_chunks <= 1) {
-    hipLaunchKernelGGL((delta_rule_kernel<T, CPT, false>),
+    hipLaunchKernelGGL((delta_rule_kernel<T, CPT, false, CH>),
                        dim3(n_seqs, A.heads, vz), dim3(256), lds, st, out, A,
                        state, slots, cu_q, ctx_lens, 0, 0, 1, nullptr);
     return;
   }
   const int vz1 = (Dv + D + VS - 1) / VS;
-  hipLaunchKernelGGL((delta_rule_kernel<T, CPT, true>),
+  hipLaunchKernelGGL((delta_rule_kernel<T, CPT, true, CH>),
                      dim3(n_seqs * max_chunks, A.heads, vz1), dim3(256), lds,
                      st, out, A, state, slots, cu_q, ctx_lens, 1, chunk,
                      max_chunks, ws);
@@ -514,32 +538,29 @@ void launch_delta_rule_cpt(float* out, const DRArgs<T>& A, float* state,
   else if (n_tiles <= 8) DR_SCAN(8);
   else DR_SCAN(16);
 #undef DR_SCAN
-  hipLaunchKernelGGL((delta_rule_kernel<T, CPT, false>),
+  hipLaunchKernelGGL((delta_rule_kernel<T, CPT, false, CH>),
                      dim3(n_seqs * max_chunks, A.heads, vz), dim3(256), lds,
                      st, out, A, state, slots, cu_q, ctx_lens, 2, chunk,
                      max_chunks, ws);
 }
 
-template <typename T>
-void launch_delta_rule(float* out, const T* q, const T* k, const T* v,
-                       const T* b, const T* a, long q_stride, long k_stride,
-                       long v_stride, long b_stride, long a_stride,
-                       const float* dt_bias, const float* A_log, float* state,
-                       const int* slots, const int* cu_q, const int* ctx_lens,
-                       int n_seqs, int heads, int groups, int D, int Dv,
-                       int chunk, int max_chunks, float* ws, hipStream_t st) {
-  if (n_seqs == 0) return;
-  DRArgs<T> A{q, k, v, b, a, q_stride, k_stride, v_stride, b_stride, a_stride,
-              dt_bias, A_log, heads, groups, D, Dv};
+template <typename T, bool CH>
+void launch_delta_rule_as(float* out, const DRArgs<T>& A, float* state,
+                          const int* slots, const int* cu_q,
+                          const int* ctx_lens, int n_seqs, int chunk,
+                          int max_chunks, float* ws, hipStream_t st) {
+  const int D = A.D, Dv = A.Dv, heads = A.heads;
   if (cu_q == nullptr && Dv % 4 == 0 && Dv <= 1024) {
     const int RG = 256 / (Dv / 4);
     const int nr = RG >= 1 ? (D + RG - 1) / RG : 0;
     const size_t l2 =
-        (size_t)(2 * ((D + 3) & ~3) + Dv + 2 * RG * Dv) * sizeof(float);
+        (size_t)(2 * ((D + 3) & ~3) + Dv + 2 * RG * Dv + (CH ? D : 0)) *
+        sizeof(float);
     if (RG >= 1 && nr <= 32 && l2 <= 64 * 1024) {
 #define DR_DEC(NR)                                                            \
-  hipLaunchKernelGGL((delta_rule_decode_kernel<T, NR>), dim3(n_seqs, heads),  \
-                     dim3(256), l2, st, out, A, state, slots, ctx_lens)
+  hipLaunchKernelGGL((delta_rule_decode_kernel<T, NR, CH>),                   \
+                     dim3(n_seqs, heads), dim3(256), l2, st, out, A, state,   \
+                     slots, ctx_lens)
       if (nr <= 4) DR_DEC(4);
       else if (nr <= 8) DR_DEC(8);
       else if (nr <= 16) DR_DEC(16);
@@ -554,17 +575,37 @@ void launch_delta_rule(float* out, const T* q, const T* k, const T* v,
       (long)n_seqs * max_chunks * heads * ((Dv + 63) / 64) >= 256;
   if (const char* e = std::getenv("XLLM_DELTA_COLS")) wide = e[0] == '4';
   if (wide)
-    launch_delta_rule_cpt<T, 4>(out, A, state, slots, cu_q, ctx_lens, n_seqs,
-                                chunk, max_chunks, ws, st);
+    launch_delta_rule_cpt<T, 4, CH>(out, A, state, slots, cu_q, ctx_lens,
+                                    n_seqs, chunk, max_chunks, ws, st);
   else
-    launch_delta_rule_cpt<T, 1>(out, A, state, slots, cu_q, ctx_lens, n_seqs,
-                                chunk, max_chunks, ws, st);
+    launch_delta_rule_cpt<T, 1, CH>(out, A, state, slots, cu_q, ctx_lens,
+                                    n_seqs, chunk, max_chunks, ws, st);
+}
+
+template <typename T>
+void launch_delta_rule(float* out, const T* q, const T* k, const T* v,
+                       const T* b, const T* a, long q_stride, long k_stride,
+                       long v_stride, long b_stride, long a_stride,
+                       const float* dt_bias, const float* A_log,
+                       int channel_decay, float* state, const int* slots,
+                       const int* cu_q, const int* ctx_lens, int n_seqs,
+                       int heads, int groups, int D, int Dv, int chunk,
+                       int max_chunks, float* ws, hipStream_t st) {
+  if (n_seqs == 0) return;
+  const DRArgs<T> A{q, k, v, b, a, q_stride, k_stride, v_stride, b_stride,
+                    a_stride, dt_bias, A_log, heads, groups, D, Dv};
+  if (channel_decay)
+    launch_delta_rule_as<T, true>(out, A, state, slots, cu_q, ctx_lens,
+                                  n_seqs, chunk, max_chunks, ws, st);
+  else
+    launch_delta_rule_as<T, false>(out, A, state, slots, cu_q, ctx_lens,
+                                   n_seqs, chunk, max_chunks, ws, st);
 }
 
 #define INST_DR(T)                                                            \
   template void launch_delta_rule<T>(                                         \
       float*, const T*, const T*, const T*, const T*, const T*, long, long,   \
-      long, long, long, const float*, const float*, float*, const int*,       \
+      long, long, long, const float*, const float*, int, float*, const int*,  \
       const int*, const int*, int, int, int, int, int, int, int, float*,      \
       hipStream_t);
 INST_DR(float)

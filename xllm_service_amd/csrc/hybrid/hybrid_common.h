@@ -25,5 +25,30 @@ template <> struct IO<unsigned short> {
 XLLM_DEV float sigmoidf_(float x) { return 1.0f / (1.0f + __expf(-x)); }
 XLLM_DEV float siluf_(float x) { return x / (1.0f + __expf(-x)); }
 
+// four neighbouring values at once (16 B of fp32, 8 B of bf16)
+template <typename T> struct Quad;
+template <> struct Quad<float> {
+  static XLLM_DEV void ld(const float* p, float v[4]) {
+    const float4 x = *reinterpret_cast<const float4*>(p);
+    v[0] = x.x; v[1] = x.y; v[2] = x.z; v[3] = x.w;
+  }
+  static XLLM_DEV void st(float* p, const float v[4]) {
+    *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+  }
+};
+template <> struct Quad<unsigned short> {
+  static XLLM_DEV void ld(const unsigned short* p, float v[4]) {
+    const ushort4_t x = *reinterpret_cast<const ushort4_t*>(p);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = bf16_to_f32(x.x[i]);
+  }
+  static XLLM_DEV void st(unsigned short* p, const float v[4]) {
+    ushort4_t x;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) x.x[i] = f32_to_bf16(v[i]);
+    *reinterpret_cast<ushort4_t*>(p) = x;
+  }
+};
+
 }  // namespace hyb
 }  // namespace xllm

@@ -6,6 +6,7 @@
 // cached row. Values are the latent itself (first kv_rank entries of the
 // row); the value up-projection is applied by the caller afterwards.
 //
+// With a window a query sees only the last `window` keys, itself included.
 // Scores, softmax weights and the weighted sum are fp32. One wavefront per
 // (query token, head): 64 keys are scored per step, one per lane, then the
 // lanes switch to owning output columns for the weighted sum.
@@ -14,7 +15,8 @@
 namespace xllm {
 namespace hyb {
 
-// cache row write: c = rmsnorm(dkv[:r]) * w ; kr = rope(dkv[r:]).
+// cache row write: c = rmsnorm(dkv[:r]) * w ; kr = rope(dkv[r:]), turning
+// entries 2i and 2i+1 together or, with `halves`, i and i + rot_dims/2.
 // One wavefront per token.
 template <typename T>
 __global__ void latent_kv_store_kernel(
@@ -22,7 +24,7 @@ __global__ void latent_kv_store_kernel(
     const float* __restrict__ norm_w, float eps,
     const long* __restrict__ pos, const double* __restrict__ inv_freq,
     float mscale, int rot_dims, const long* __restrict__ slots, int r, int rd,
-    long dkv_stride) {
+    long dkv_stride, int halves) {
   const int t = blockIdx.x;
   const long slot = slots[t];
   if (slot < 0) return;
@@ -43,10 +45,11 @@ __global__ void latent_kv_store_kernel(
     double s, c;
     sincos((double)pos[t] * inv_freq[i], &s, &c);
     const float cf = (float)c * mscale, sf = (float)s * mscale;
-    const float u = IO<T>::ld(src + r + 2 * i);
-    const float v = IO<T>::ld(src + r + 2 * i + 1);
-    IO<T>::st(dst + r + 2 * i, u * cf - v * sf);
-    IO<T>::st(dst + r + 2 * i + 1, v * cf + u * sf);
+    const int a = r + (halves ? i : 2 * i), b = a + (halves ? half : 1);
+    const float u = IO<T>::ld(src + a);
+    const float v = IO<T>::ld(src + b);
+    IO<T>::st(dst + a, u * cf - v * sf);
+    IO<T>::st(dst + b, v * cf + u * sf);
   }
   for (int i = rot_dims + lane; i < rd; i += 64)
     IO<T>::st(dst + r + i, IO<T>::ld(src + r + i));
@@ -64,7 +67,7 @@ __global__ void latent_attn_kernel(
     const T* __restrict__ cache, const int* __restrict__ block_tables,
     const int* __restrict__ cu_q, const int* __restrict__ seq_lens,
     int n_seqs, int heads, int r, int rd, int block_size, int table_width,
-    float scale, long q_row_stride) {
+    float scale, long q_row_stride, int window) {
   extern __shared__ float smem[];
   const int W = r + rd;
   const int t = blockIdx.x;
@@ -101,7 +104,8 @@ __global__ void latent_attn_kernel(
   for (int i = 0; i < LAT_MAX_ACC; ++i) acc[i] = 0.f;
   const int n_acc = (r + 63) >> 6;
 
-  for (int k0 = 0; k0 < n_keys; k0 += 64) {
+  const int k_first = window > 0 ? max(0, n_keys - window) : 0;
+  for (int k0 = k_first; k0 < n_keys; k0 += 64) {
     const int key = k0 + lane;
     float sc = -INFINITY;
     if (key < n_keys) {
@@ -112,8 +116,8 @@ __global__ void latent_attn_kernel(
       sc = d;
     }
     const float m_new = fmaxf(m, wave_reduce_max(sc));
-    const float alpha = __expf(m - m_new);       // m=-inf first: exp(-inf)=0
-    const float p = (key < n_keys) ? __expf(sc - m_new) : 0.f;
+    const float alpha = expf(m - m_new);         // m=-inf first: exp(-inf)=0
+    const float p = (key < n_keys) ? expf(sc - m_new) : 0.f;
     l = l * alpha + wave_reduce_sum(p);
     m = m_new;
 #pragma unroll
@@ -145,11 +149,12 @@ void launch_latent_kv_store(T* cache, const T* dkv, const float* norm_w,
                             float eps, const long* pos,
                             const double* inv_freq, float mscale,
                             int rot_dims, const long* slots, int tokens,
-                            int r, int rd, long dkv_stride, hipStream_t st) {
+                            int r, int rd, long dkv_stride, int halves,
+                            hipStream_t st) {
   if (tokens == 0) return;
   hipLaunchKernelGGL((latent_kv_store_kernel<T>), dim3(tokens), dim3(64), 0,
                      st, cache, dkv, norm_w, eps, pos, inv_freq, mscale,
-                     rot_dims, slots, r, rd, dkv_stride);
+                     rot_dims, slots, r, rd, dkv_stride, halves);
 }
 
 template <typename T>
@@ -158,7 +163,7 @@ void launch_latent_attn(float* out, const T* q, const T* cache,
                         const int* seq_lens, int tokens, int n_seqs,
                         int heads, int r, int rd, int block_size,
                         int table_width, float scale, long q_row_stride,
-                        hipStream_t st) {
+                        int window, hipStream_t st) {
   if (tokens == 0) return;
   const int nw = heads < 4 ? heads : 4;
   const int W = r + rd;
@@ -166,17 +171,17 @@ void launch_latent_attn(float* out, const T* q, const T* cache,
   hipLaunchKernelGGL((latent_attn_kernel<T>), grid, dim3(64 * nw),
                      (size_t)nw * W * sizeof(float), st, out, q, cache,
                      block_tables, cu_q, seq_lens, n_seqs, heads, r, rd,
-                     block_size, table_width, scale, q_row_stride);
+                     block_size, table_width, scale, q_row_stride, window);
 }
 
 #define INST_LAT(T)                                                          \
   template void launch_latent_kv_store<T>(                                   \
       T*, const T*, const float*, float, const long*, const double*, float,  \
-      int, const long*, int, int, int, long, hipStream_t);                   \
+      int, const long*, int, int, int, long, int, hipStream_t);              \
   template void launch_latent_attn<T>(float*, const T*, const T*,            \
                                       const int*, const int*, const int*,    \
                                       int, int, int, int, int, int, int,     \
-                                      float, long, hipStream_t);
+                                      float, long, int, hipStream_t);
 INST_LAT(float)
 INST_LAT(unsigned short)
 

@@ -30,6 +30,9 @@
 // Decode splits the context over `n_part` workgroups per token; partial
 // (acc, max, sum) triples are merged by a second small kernel.
 //
+// Sliding window: a row sees the keys [limit - window, limit); the tile loop
+// starts at the first tile any row of the workgroup needs.
+//
 // Fragment layouts of __builtin_amdgcn_mfma_f32_16x16x32_bf16 (lane l):
 //   A[l&15][(l>>4)*8 + j], B[(l>>4)*8 + j][l&15], C[(l>>4)*4 + r][l&15].
 #include "hybrid_common.h"
@@ -60,7 +63,7 @@ __global__ void __launch_bounds__(256) latent_attn_mfma_kernel(
     const unsigned short* __restrict__ cache,
     const int* __restrict__ block_tables, const int* __restrict__ cu_q,
     const int* __restrict__ seq_lens, int n_seqs, int heads, int r, int rd,
-    int block_size, int table_width, float scale, int n_part) {
+    int block_size, int table_width, float scale, int n_part, int window) {
   extern __shared__ unsigned short vt[];          // tr16 image, see above
   __shared__ int tbl[512];                        // block ids of this key range
   constexpr int RT = 4 / CS;                      // row tiles per workgroup
@@ -98,8 +101,11 @@ __global__ void __launch_bounds__(256) latent_attn_mfma_kernel(
   const int last_row = min(row0 + ROWS_WG, rows_in_seq) - 1;
   const int kmax = ctx + last_row / heads + 1;       // keys any row here sees
   const int n_tiles = (kmax + LM_KT - 1) / LM_KT;
-  const int tpp = (n_tiles + n_part - 1) / n_part;
-  const int t_begin = blockIdx.y * tpp;
+  // first tile with a key the earliest row of this workgroup sees
+  const int t_first =
+      window > 0 ? max(0, ctx + row0 / heads + 1 - window) / LM_KT : 0;
+  const int tpp = (n_tiles - t_first + n_part - 1) / n_part;
+  const int t_begin = t_first + blockIdx.y * tpp;
   const int t_end = min(n_tiles, t_begin + tpp);
   const int* table = block_tables + (long)s * table_width;
 
@@ -109,6 +115,7 @@ __global__ void __launch_bounds__(256) latent_attn_mfma_kernel(
   const bool wave_on = row0 + rt * 16 < rows_in_seq;
   const bool row_ok = rho < rows_in_seq;
   const int limit = row_ok ? ctx + rho / heads + 1 : 0;
+  const int lo = window > 0 ? limit - window : 0;
   const long grow = (long)q0 * heads + rho;          // row in [T*H]
 
   bf16x8 qf[KQ];
@@ -201,7 +208,8 @@ __global__ void __launch_bounds__(256) latent_attn_mfma_kernel(
 #pragma unroll
       for (int rr = 0; rr < 4; ++rr) {
         const int kk = k0 + g * 8 + h2 * 4 + rr;     // key of C row g*4+rr
-        sc[h2 * 4 + rr] = (kk < limit) ? sacc[rr] * scale : -INFINITY;
+        sc[h2 * 4 + rr] =
+            (kk < limit && kk >= lo) ? sacc[rr] * scale : -INFINITY;
       }
     }
     float mloc = sc[0];
@@ -338,7 +346,7 @@ void launch_latent_attn_mfma(float* out, float* ws_acc, float* ws_ml,
                              const int* seq_lens, int tokens, int n_seqs,
                              int heads, int r, int rd, int block_size,
                              int table_width, float scale, int n_part,
-                             hipStream_t st) {
+                             int window, hipStream_t st) {
   if (tokens == 0) return;
   const int cls = latent_attn_mfma_class(r + rd, r);
   const int rp = (r + 15) & ~15;
@@ -359,7 +367,7 @@ void launch_latent_attn_mfma(float* out, float* ws_acc, float* ws_ml,
   hipLaunchKernelGGL((latent_attn_mfma_kernel<KQ, NO, CS>), grid, dim3(256), \
                      lds, st, out, ws_acc, ws_ml, q, cache, block_tables,    \
                      cu_q, seq_lens, n_seqs, heads, r, rd, block_size,       \
-                     table_width, scale, n_part)
+                     table_width, scale, n_part, window)
 #define LM_BY_CS(KQ, NO)                                                     \
   do {                                                                       \
     if (cs == 4) LM_LAUNCH(KQ, NO, 4);                                       \

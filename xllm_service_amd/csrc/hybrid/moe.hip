@@ -101,7 +101,8 @@ __global__ void moe_route_kernel(int* __restrict__ ids,
 }
 
 // out[t, c] = sum_k wts[t, k] * y[rows[t, k], c] (+ extra[t, c]); a negative
-// row reads ident[t, c] (an expert whose output is its input). fp32 sums.
+// row reads ident[t, c] (an expert whose output is its input); without wts a
+// plain sum. fp32 sums.
 template <typename T>
 __global__ void moe_combine_kernel(float* __restrict__ out,
                                    const T* __restrict__ y,
@@ -123,7 +124,7 @@ __global__ void moe_combine_kernel(float* __restrict__ out,
       float v = 0.f;
       if (r >= 0) v = IO<T>::ld(y + (long)r * width + c);
       else if (ident != nullptr) v = IO<T>::ld(ident + t * ident_stride + c);
-      a += wts[t * top + kk] * v;
+      a += wts != nullptr ? wts[t * top + kk] * v : v;
     }
     if (extra != nullptr) a += IO<T>::ld(extra + t * extra_stride + c);
     out[idx] = a;

@@ -195,14 +195,16 @@ __global__ void act_mul_kernel(T* __restrict__ out, const T* __restrict__ x,
 }
 
 // Rotate pairs (2i, 2i+1), i < rot_dims/2, of x[t, h, off : off+rot_dims] by
-// pos[t] * inv_freq[i] (angle in fp64), cos/sin scaled by mscale. In place.
+// pos[t] * inv_freq[i] (angle in fp64), cos/sin scaled by mscale; with
+// `halves` entry i turns with entry i + rot_dims/2. In place.
 template <typename T>
 __global__ void rope_interleaved_kernel(T* __restrict__ x,
                                         const long* __restrict__ pos,
                                         const double* __restrict__ inv_freq,
                                         float mscale, int tokens, int heads,
                                         int half, long row_stride,
-                                        long head_stride, int off) {
+                                        long head_stride, int off,
+                                        int halves) {
   const long n = (long)tokens * heads * half;
   for (long idx = blockIdx.x * (long)blockDim.x + threadIdx.x; idx < n;
        idx += (long)gridDim.x * blockDim.x) {
@@ -213,10 +215,11 @@ __global__ void rope_interleaved_kernel(T* __restrict__ x,
     double s, c;
     sincos((double)pos[t] * inv_freq[i], &s, &c);
     const float cf = (float)c * mscale, sf = (float)s * mscale;
-    T* p = x + t * row_stride + h * head_stride + off + 2 * i;
-    const float u = IO<T>::ld(p), v = IO<T>::ld(p + 1);
+    T* p = x + t * row_stride + h * head_stride + off + (halves ? i : 2 * i);
+    T* p2 = p + (halves ? half : 1);
+    const float u = IO<T>::ld(p), v = IO<T>::ld(p2);
     IO<T>::st(p, u * cf - v * sf);
-    IO<T>::st(p + 1, v * cf + u * sf);
+    IO<T>::st(p2, v * cf + u * sf);
   }
 }
 
@@ -288,13 +291,13 @@ template <typename T>
 void launch_rope_interleaved(T* x, const long* pos, const double* inv_freq,
                              float mscale, int tokens, int heads, int half,
                              long row_stride, long head_stride, int off,
-                             hipStream_t st) {
+                             int halves, hipStream_t st) {
   const long n = (long)tokens * heads * half;
   if (n == 0) return;
   const int blocks = (int)((n + 255) / 256 < 65535 ? (n + 255) / 256 : 65535);
   hipLaunchKernelGGL((rope_interleaved_kernel<T>), dim3(blocks), dim3(256), 0,
                      st, x, pos, inv_freq, mscale, tokens, heads, half,
-                     row_stride, head_stride, off);
+                     row_stride, head_stride, off, halves);
 }
 
 #define INST_NORMS(T)                                                         \
@@ -309,7 +312,7 @@ void launch_rope_interleaved(T* x, const long* pos, const double* inv_freq,
                                            int, int, int, int, hipStream_t);  \
   template void launch_rope_interleaved<T>(T*, const long*, const double*,    \
                                            float, int, int, int, long, long,  \
-                                           int, hipStream_t);
+                                           int, int, hipStream_t);
 INST_NORMS(float)
 INST_NORMS(unsigned short)
 

@@ -5,7 +5,7 @@
 //   (u, v) -> (u cos a - v sin a, v cos a + u sin a),  a = pos * f_i,
 // with the pair (u, v) = entries (2i, 2i+1) of the head (`pairs`) or entries
 // (i, i + rot/2); then, with `unit`, the head is divided by its root mean
-// square sqrt(mean(x^2) + eps). Angle and sincos in fp64, the turn and the
+// square sqrt(mean(x^2) + eps). cos and sin carry the factor mscale. Angle and sincos in fp64, the turn and the
 // norm in fp32. q' goes to a contiguous row tensor, k' and the untouched v
 // (when there is one) into the paged caches [blocks, n_kv, block, D | Dv] at
 // the token's slot (slot < 0: not stored). One workgroup per token; cos/sin
@@ -30,7 +30,7 @@ __global__ void __launch_bounds__(256) rope_headnorm_store_kernel(
     const long* __restrict__ pos, const double* __restrict__ inv_freq, int rot,
     int pairs, int unit, float eps, int heads, int n_kv, int D, int Dv,
     T* __restrict__ k_cache, T* __restrict__ v_cache,
-    const long* __restrict__ slot_mapping, int block_size) {
+    const long* __restrict__ slot_mapping, int block_size, float mscale) {
   extern __shared__ float cs[];           // [rot/2] cos, [rot/2] sin
   const int t = blockIdx.x, tid = threadIdx.x;
   const int lane = tid & 63, wv = tid >> 6;
@@ -38,8 +38,8 @@ __global__ void __launch_bounds__(256) rope_headnorm_store_kernel(
   for (int i = tid; i < half; i += 256) {
     double s, c;
     sincos((double)pos[t] * inv_freq[i], &s, &c);
-    cs[i] = (float)c;
-    cs[half + i] = (float)s;
+    cs[i] = (float)(c * mscale);
+    cs[half + i] = (float)(s * mscale);
   }
   __syncthreads();
   const long slot = slot_mapping[t];
@@ -148,13 +148,13 @@ void launch_rope_headnorm_store(T* q_out, const T* q, const T* k, const T* v,
                                 int tokens, int heads, int n_kv, int D, int Dv,
                                 T* k_cache, T* v_cache,
                                 const long* slot_mapping, int block_size,
-                                hipStream_t st) {
+                                float mscale, hipStream_t st) {
   if (tokens == 0) return;
   hipLaunchKernelGGL((rope_headnorm_store_kernel<T>), dim3(tokens), dim3(256),
                      (size_t)(rot > 0 ? rot : 1) * sizeof(float), st, q_out, q,
                      k, v, q_stride, k_stride, v_stride, pos, inv_freq, rot,
                      pairs, unit, eps, heads, n_kv, D, Dv, k_cache, v_cache,
-                     slot_mapping, block_size);
+                     slot_mapping, block_size, mscale);
 }
 
 template <typename T>
@@ -179,7 +179,7 @@ void launch_gelu_tanh_gate(T* out, const T* g, const T* u, long rows, int F,
   template void launch_rope_headnorm_store<T>(                                \
       T*, const T*, const T*, const T*, long, long, long, const long*,        \
       const double*, int, int, int, float, int, int, int, int, int, T*, T*,   \
-      const long*, int, hipStream_t);                                         \
+      const long*, int, float, hipStream_t);                                  \
   template void launch_polynorm<T>(T*, const T*, const float*, float, long,   \
                                    int, long, hipStream_t);                   \
   template void launch_gelu_tanh_gate<T>(T*, const T*, const T*, long, int,   \

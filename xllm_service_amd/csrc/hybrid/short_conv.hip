@@ -14,8 +14,13 @@
 // to a row-major tensor or straight into a paged cache
 // [blocks, heads, block, hd] at the token's slot.
 //
+// With add_input the result is u[t, c] + y[t, c] (the input beside its
+// convolution).
+//
 // A second kernel moves the state forward once every reader of the old state
-// has been launched (same stream).
+// has been launched (same stream). For decode rows (one token per sequence)
+// the convolution can do it itself (`advance`): a channel's state is read and
+// written by one thread only.
 #include "hybrid_common.h"
 
 namespace xllm {
@@ -40,11 +45,12 @@ __global__ void __launch_bounds__(256) short_conv_kernel(
     T* __restrict__ out, long out_stride, T* __restrict__ cache,
     const long* __restrict__ slot_mapping, int block_size,
     const T* __restrict__ x, long x_stride, const T* __restrict__ w,
-    const T* __restrict__ bias, const T* __restrict__ state, long state_row,
+    const T* __restrict__ bias, T* state, long state_row,
     int state_off, const int* __restrict__ slots, const int* __restrict__ cu_q,
     const int* __restrict__ ctx_lens, int n_seqs, int heads, int hd, int taps,
     int act_silu, int rot_dims, const long* __restrict__ pos,
-    const double* __restrict__ inv_freq, int tokens, int tile) {
+    const double* __restrict__ inv_freq, int tokens, int tile, int add_input,
+    int advance) {
   const int ppairs = (hd + 1) >> 1;
   const int idx = blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= heads * ppairs) return;
@@ -117,6 +123,24 @@ __global__ void __launch_bounds__(256) short_conv_kernel(
         if (two) a1 += IO<T>::ld(w + (long)(c0 + 1) * taps + jj) * u1;
       }
     }
+    if (advance && slot >= 0) {            // decode: taps 1.. become the state
+      T* st = state + (long)slot * K1 * state_row + state_off + c0;
+      if (TAPS > 0) {
+#pragma unroll
+        for (int jj = 0; jj < NT - 1; ++jj) {
+          IO<T>::st(st + (long)jj * state_row, h0[jj + 1]);
+          if (two) IO<T>::st(st + (long)jj * state_row + 1, h1[jj + 1]);
+        }
+      } else {
+        for (int jj = 0; jj < K1; ++jj) {  // ascending: reads run ahead
+          const T* src = jj + 1 < K1 ? st + (long)(jj + 1) * state_row
+                                     : x + (long)t * x_stride + c0;
+          const T v0 = src[0], v1 = two ? src[1] : v0;
+          st[(long)jj * state_row] = v0;
+          if (two) st[(long)jj * state_row + 1] = v1;
+        }
+      }
+    }
     if (act_silu) { a0 = siluf_(a0); a1 = siluf_(a1); }
     if (two && d0 + 1 < rot_dims) {
       double sn, cs;
@@ -125,6 +149,11 @@ __global__ void __launch_bounds__(256) short_conv_kernel(
       const float u = a0, v = a1;
       a0 = u * cf - v * sf;
       a1 = v * cf + u * sf;
+    }
+    if (add_input) {
+      const T* row = x + (long)t * x_stride + c0;
+      a0 += IO<T>::ld(row);
+      if (two) a1 += IO<T>::ld(row + 1);
     }
     T* dst;
     if (cache) {
@@ -168,11 +197,12 @@ template <typename T>
 void launch_short_conv(T* out, long out_stride, T* cache,
                        const long* slot_mapping, int block_size, const T* x,
                        long x_stride, const T* w, const T* bias,
-                       const T* state, long state_row, int state_off,
+                       T* state, long state_row, int state_off,
                        const int* slots, const int* cu_q, const int* ctx_lens,
                        int tokens, int n_seqs, int heads, int hd, int taps,
                        int act_silu, int rot_dims, const long* pos,
-                       const double* inv_freq, hipStream_t st) {
+                       const double* inv_freq, int add_input, int advance,
+                       hipStream_t st) {
   if (tokens == 0 || heads * hd == 0) return;
   const int n = heads * ((hd + 1) / 2);
   const int bx = n >= 256 ? 256 : ((n + 63) / 64) * 64;
@@ -185,7 +215,7 @@ void launch_short_conv(T* out, long out_stride, T* cache,
                      out_stride, cache, slot_mapping, block_size, x, x_stride, \
                      w, bias, state, state_row, state_off, slots, cu_q,       \
                      ctx_lens, n_seqs, heads, hd, taps, act_silu, rot_dims,   \
-                     pos, inv_freq, tokens, tile)
+                     pos, inv_freq, tokens, tile, add_input, advance)
   switch (taps) {
     case 2: SC_LAUNCH(2); break;
     case 3: SC_LAUNCH(3); break;
@@ -210,8 +240,8 @@ void launch_short_conv_state(T* state, long state_row, const T* x,
 #define INST_SC(T)                                                            \
   template void launch_short_conv<T>(                                         \
       T*, long, T*, const long*, int, const T*, long, const T*, const T*,     \
-      const T*, long, int, const int*, const int*, const int*, int, int, int, \
-      int, int, int, int, const long*, const double*, hipStream_t);           \
+      T*, long, int, const int*, const int*, const int*, int, int, int,       \
+      int, int, int, int, const long*, const double*, int, int, hipStream_t); \
   template void launch_short_conv_state<T>(T*, long, const T*, long,          \
                                            const int*, const int*, int, int,  \
                                            int, hipStream_t);
