@@ -366,7 +366,7 @@ def make_weights(cfg, seed=0, ranks=(3, 4)):
         return (torch.randn(*shape, generator=gen) * std).bfloat16().float()
 
     def about(mean, *shape, spread=0.2):
-        return (mean + spread * torch.randn(*shape, generator=gen)) \
+        return (mean + spread * torch.randn(shape, generator=gen)) \
             .bfloat16().float()
 
     out = {"embed": rnd(cfg["vocab"], W, std=1.0), "embed.norm": about(1.0),
