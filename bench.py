@@ -67,7 +67,8 @@ def parse_args():
                          "measurement, not the headline record)")
     ap.add_argument("--hybrid-sizes", default="2k,4k")
     ap.add_argument("--hybrid-family", default="pugovik",
-                    choices=("pugovik", "dunusun", "tosipel", "gararax"),
+                    choices=("pugovik", "dunusun", "tosipel", "gararax",
+                             "nikedra"),
                     help="which hybrid stack --mode hybrid measures beside "
                          "the equal-size llama stack")
     ap.add_argument("--model", default="llama-3-8b")
@@ -728,6 +729,205 @@ def _gararax_kernels(size, device, T, batch, ctx):
     return out
 
 
+def _nikedra_kernels(size, device, T, batch, ctx):
+    """Achieved rates of the Nikedra kernels at one layer's shapes, each
+    beside the like kernel of the tosipel / dunusun / pugovik stacks of that
+    size."""
+    from xllm_service_amd.models.config import get_config
+    from xllm_service_amd.ops import hybrid as hops
+    nc, tc, dc, pc = (get_config(f"{f}-{size}") for f in (
+        "nikedra", "tosipel", "dunusun", "pugovik"))
+
+    def mixer(cfg, kind):
+        return next(l.mixer for l in cfg.layers if l.type == kind)
+    left, ssm = mixer(nc, "parallel")["left"], mixer(nc, "parallel")["right"]
+    lat, dl = mixer(nc, "latent_attention"), mixer(nc, "channel_delta")
+    tatt, tdl = mixer(tc, "attention"), mixer(tc, "delta")
+    plat, dssm = mixer(pc, "latent_attention"), mixer(dc, "mamba2")
+    bf = dict(dtype=torch.bfloat16, device=device)
+    f32 = dict(dtype=torch.float32, device=device)
+    i32 = dict(dtype=torch.int32, device=device)
+    out = []
+    nblk = (max(T, ctx) + 15) // 16
+    tab = torch.arange(batch * nblk, **i32).view(batch, nblk)
+    cu = torch.tensor([0, T], **i32)
+    sl = torch.tensor([T], **i32)
+    sld = torch.full((batch,), ctx, **i32)
+    z1 = torch.zeros(1, **i32)
+    sls = torch.arange(batch, **i32)
+
+    def add(label, fn, work, unit, iters=10):
+        t = _time_gpu(fn, iters, 3)
+        out.append((label, t, work / t / (1e12 if "FLOP" in unit else 1e9),
+                    unit))
+    # ---- chunked attention vs windowed attention ---------------------------
+    for label, m, chunked in (("chunk attn", left, True),
+                              ("window+sink attn (tosipel)", tatt, False)):
+        H, G, D, Dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        win = m["mask"]["size"]
+        kc = torch.randn(batch * nblk, G, 16, D, **bf)
+        vc = torch.randn(batch * nblk, G, 16, Dv, **bf)
+        q = torch.randn(T, H * D, **bf)
+        o = torch.empty(T, H, Dv, **f32)
+        kw = dict(window=win, chunked=chunked,
+                  sink=None if chunked else torch.zeros(H, **f32))
+        seen = sum(i % win + 1 if chunked else min(i + 1, win)
+                   for i in range(T))
+        add(f"{label} prefill ({win})",
+            lambda: hops.capped_attn(q, kc, vc, tab[:1], cu, sl, H,
+                                     m["scale"], 0.0, o, **kw),
+            2.0 * H * (D + Dv) * seen, "TFLOP/s", 3)
+        qd = torch.randn(batch, H * D, **bf)
+        od = torch.empty(batch, H, Dv, **f32)
+        keys = (ctx - 1) % win + 1 if chunked else min(ctx, win)
+        add(f"{label} decode ({win})",
+            lambda: hops.capped_attn(qd, kc, vc, tab, None, sld, H,
+                                     m["scale"], 0.0, od, **kw),
+            batch * keys * G * (D + Dv) * 2, "GB/s")
+        del kc, vc
+    # ---- latent attention with and without a window ------------------------
+    for label, m, win in (("latent window attn", lat, lat["mask"]["size"]),
+                          ("latent_attn (pugovik)", plat, 0)):
+        H, r, W = m["heads"], m["kv_rank"], m["kv_rank"] + m["rot_dim"]
+        cache = torch.randn(batch * nblk, 16, W, **bf)
+        q = torch.randn(T, H, W, **bf)
+        o = torch.empty(T, H, r, **f32)
+        seen = sum(min(i + 1, win or T) for i in range(T))
+        add(f"{label} prefill",
+            lambda: hops.latent_attn(q, cache, tab[:1], cu, sl, 0.1, r, o,
+                                     win),
+            2.0 * H * (W + r) * seen, "TFLOP/s", 3)
+        qd = torch.randn(batch, H, W, **bf)
+        od = torch.empty(batch, H, r, **f32)
+        add(f"{label} decode",
+            lambda: hops.latent_attn(qd, cache, tab, None, sld, 0.1, r, od,
+                                     win),
+            batch * min(ctx, win or ctx) * W * 2, "GB/s")
+    # ---- delta rule, channel decays vs head decays -------------------------
+    for label, m, ch in (("channel delta_rule", dl, True),
+                         ("delta_rule (tosipel)", tdl, False)):
+        H, G, D, Dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        n = H * D if ch else H
+        st = torch.zeros(batch, H, D, Dv, **f32)
+        dtb, al = torch.zeros(n, **f32), torch.zeros(H, **f32)
+        for tokens, slots, cuq, ctxl, tail in (
+                (T, z1, cu, z1, "prefill"), (batch, sls, None, sld, "decode")):
+            qq = torch.randn(tokens, G * D, **bf)
+            vv = torch.randn(tokens, H * Dv, **bf)
+            bb, aa = torch.randn(tokens, H, **bf), torch.randn(tokens, n, **bf)
+            oo = torch.empty(tokens, H, Dv, **f32)
+            work = 8.0 * H * D * Dv * T if cuq is not None \
+                else batch * H * D * Dv * 8
+            add(f"{label} {tail}",
+                lambda: hops.delta_rule(qq, qq, vv, bb, aa, dtb, al, st,
+                                        slots, cuq, ctxl, G, oo,
+                                        max_q_len=tokens), work,
+                "GB/s" if cuq is None else "TFLOP/s (recurrence form)",
+                10 if cuq is None else 3)
+    # ---- state space recurrence ---------------------------------------------
+    for label, m in (("state space", ssm), ("state space (dunusun)", dssm)):
+        H, P, N, G = m["heads"], m["vdim"], m["state"], m["groups"]
+        st = torch.zeros(batch, H, N, P, **f32)
+        p0 = torch.zeros(H, **f32)
+        for tokens, slots, cuq, ctxl, tail in (
+                (T, z1, cu, z1, "prefill"), (batch, sls, None, sld, "decode")):
+            qq = torch.randn(tokens, G * N, **bf)
+            vv, gg = torch.randn(tokens, H * P, **bf), \
+                torch.randn(tokens, H, **bf)
+            oo = torch.empty(tokens, H, P, **f32)
+            work = 4.0 * H * N * P * T if cuq is not None \
+                else batch * H * N * P * 8
+            add(f"{label} {tail}",
+                lambda: hops.gated_recurrence(
+                    0, qq, qq, vv, gg, p0, p0, p0, 0.0, 1.0, st, slots, cuq,
+                    ctxl, G, oo, max_q_len=tokens), work,
+                "GB/s" if cuq is None else "TFLOP/s (recurrence form)",
+                10 if cuq is None else 3)
+    # ---- input convolution ----------------------------------------------------
+    Wd = nc.hidden_size
+    xin = torch.randn(T, Wd, **bf)
+    cw = torch.randn(Wd, nc.canon_taps, **bf)
+    cst = torch.zeros(batch, nc.canon_taps - 1, Wd, **bf)
+    add("input convolution",
+        lambda: hops.short_conv(xin, cw, None, cst, 0, z1, cu, z1, 1, Wd,
+                                add_input=True, advance=True), T * Wd * 4,
+        "GB/s")
+    add("short_conv+silu (dunusun, tosipel)",
+        lambda: hops.short_conv(xin, cw, None, cst, 0, z1, cu, z1, 1, Wd,
+                                act_silu=True), T * Wd * 4, "GB/s")
+    xd = xin[:batch].contiguous()
+    add(f"input convolution + state, {batch} rows (decode)",
+        lambda: hops.short_conv(xd, cw, None, cst, 0, sls, None, sld, 1, Wd,
+                                add_input=True, advance=True),
+        batch * Wd * 2 * (2 + 2 * (nc.canon_taps - 1)), "GB/s")
+    # ---- depth average vs the streams kernel ----------------------------------
+    lv = nc.num_layers
+    w, g = torch.ones(Wd, **f32), torch.ones(1, **f32)
+    for rows, tail in ((T, ""), (batch, f", {batch} rows (decode)")):
+        hist = torch.randn(lv + 1, rows, Wd, **f32)
+        x, m1 = torch.randn(rows, Wd, **f32), torch.randn(rows, Wd, **bf)
+        for level in (1, lv):
+            dwa = torch.ones(level + 1, **f32)
+            add(f"depth_mix_norm, level {level}{tail}",
+                lambda: hops.depth_mix_norm(
+                    x, hist, level, m1, None, None, None, 1.0, m1, dwa, g, g,
+                    1e-6, torch.bfloat16, x),
+                rows * Wd * (4 * (level + 3) + 2 * 4), "GB/s")
+        dwa = torch.ones(lv + 1, **f32)
+        add(f"depth_mix_norm, level {lv}, two normed halves{tail}",
+            lambda: hops.depth_mix_norm(
+                x, hist, lv, m1, w, m1, w, 0.5, x, dwa, g, g, 1e-6,
+                torch.bfloat16, x), rows * Wd * (4 * (lv + 4) + 2 * 4),
+            "GB/s")
+        S = dc.streams or 1
+        xs = torch.randn(rows, S, Wd, **f32)
+        wi, mix = torch.ones(S, **f32), torch.eye(S, **f32)
+        add(f"streams_update_mix_norm (dunusun){tail}",
+            lambda: hops.streams_update_mix_norm_(
+                xs, mix, wi, m1, 1.0, m1, 1.0, wi, w, w, 1e-6),
+            rows * Wd * (8 * S + 6), "GB/s")
+    # ---- query/key preparation, gates, experts --------------------------------
+    H, G, D, Dv = left["heads"], left["kv_heads"], left["dim"], left["vdim"]
+    rot = left["rot"]["dims"]
+    proj = torch.randn(T, H * D + G * D + G * Dv, **bf)
+    kc = torch.zeros(nblk, G, 16, D, **bf)
+    vc = torch.zeros(nblk, G, 16, Dv, **bf)
+    pos = torch.arange(T, dtype=torch.long, device=device)
+    inv = torch.rand(rot // 2, dtype=torch.float64, device=device)
+    wq, wk = torch.ones(H * D, **f32), torch.ones(G * D, **f32)
+    q, k, v = proj[:, :H * D], proj[:, H * D:H * D + G * D], \
+        proj[:, H * D + G * D:]
+    nb = T * (2 * H * D + 2 * G * D + 2 * G * Dv) * 2
+    add("rope_headnorm_store (half layout, multiplier)",
+        lambda: hops.rope_headnorm_store(q, k, v, pos, inv, rot, False, False,
+                                         1e-6, H, G, kc, vc, pos, 1.1), nb,
+        "GB/s")
+    add("rownorm_rope_store (tosipel)",
+        lambda: hops.rownorm_rope_store(q, k, v, wq, wk, 1e-6, pos, inv, rot,
+                                        H, G, kc, vc, pos), nb, "GB/s")
+    ff = 3 * Wd // 2
+    gu = torch.randn(T, 2 * ff, **bf)
+    add("clamped_glu", lambda: hops.clamped_glu(gu, 7.0, 1.702, 1.0),
+        T * ff * 6, "GB/s")
+    add("gelu_tanh_mul (tosipel)", lambda: hops.gelu_tanh_mul(gu),
+        T * ff * 6, "GB/s")
+    mlp = next(l.mlp for l in nc.layers if l.mlp["kind"] == "moe")
+    E, top, eff = mlp["router"]["experts"], mlp["router"]["top"], \
+        mlp["expert"]["ff"]
+    ze = torch.randn(T * top, eff, **bf)
+    sc = torch.rand(T * top, **f32)
+    add("gelu_scaled (sorted rows)", lambda: hops.gelu_scaled(ze, sc),
+        T * top * eff * 4, "GB/s")
+    add("silu_mul (pugovik)", lambda: hops.silu_mul(gu), T * ff * 6, "GB/s")
+    zd = torch.randn(E, batch, eff, **bf)
+    ids = torch.randint(0, E, (batch, top), **i32)
+    wd = torch.rand(batch, top, **f32)
+    add(f"gelu_scaled ({batch} tokens x {E} experts)",
+        lambda: hops.gelu_scaled(zd, None, ids, wd), E * batch * eff * 2,
+        "GB/s written")
+    return out
+
+
 def run_hybrid_mode(args, device):
     assert torch.cuda.is_available(), "hybrid mode measures the HIP path"
     kernels = _hybrid_kernels
@@ -741,6 +941,9 @@ def run_hybrid_mode(args, device):
     if args.hybrid_family == "gararax":
         kernels = _gararax_kernels
         fams = ("gararax", "tosipel", "pugovik", "llama")
+    if args.hybrid_family == "nikedra":
+        kernels = _nikedra_kernels
+        fams = ("nikedra", "tosipel", "dunusun", "pugovik", "llama")
     for size in args.hybrid_sizes.split(","):
         T, batch, ctx = 4096, 32, 2048
         for name, t, rate, unit in kernels(size, device, T, batch, ctx):
