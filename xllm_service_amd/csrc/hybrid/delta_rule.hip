@@ -76,19 +76,20 @@ struct DRArgs {
   int heads, groups, D, Dv;
 };
 
-// decay of token `row`: entry e of the a row, A_log of head h
+// decay of token `row` from entry e of the a row; rate = -exp(A_log) of its
+// head
 template <typename T>
-XLLM_DEV float dr_decay(const DRArgs<T>& A, long row, int h, int e) {
+XLLM_DEV float dr_decay(const DRArgs<T>& A, long row, float rate, int e) {
   const float dt = dr_softplus(IO<T>::ld(A.a + row * A.a_stride + e) +
                                A.dt_bias[e]);
-  return expf(-expf(A.A_log[h]) * dt);
+  return expf(rate * dt);
 }
 
 // decay (1 with channel decays) and write strength of token `row`, head h
 template <typename T, bool CH>
-XLLM_DEV void dr_gates(const DRArgs<T>& A, long row, int h, float* g,
-                       float* beta) {
-  *g = CH ? 1.0f : dr_decay<T>(A, row, h, h);
+XLLM_DEV void dr_gates(const DRArgs<T>& A, long row, int h, float rate,
+                       float* g, float* beta) {
+  *g = CH ? 1.0f : dr_decay<T>(A, row, rate, h);
   *beta = 1.0f / (1.0f + expf(-IO<T>::ld(A.b + row * A.b_stride + h)));
 }
 
@@ -134,6 +135,7 @@ __global__ void __launch_bounds__(256) delta_rule_kernel(
   const int slot = slots[s];
   const int M = (D + DR_R - 1) / DR_R;
   const float qmul = 1.0f / sqrtf((float)D);
+  const float rate = -expf(A.A_log[h]);
 
   float S[DR_MAXM][CPT];
 #pragma unroll
@@ -183,7 +185,7 @@ __global__ void __launch_bounds__(256) delta_rule_kernel(
       const long row = tb + tt;
       qs[idx] = IO<T>::ld(A.q + row * A.q_stride + kg * D + i);
       ks[idx] = IO<T>::ld(A.k + row * A.k_stride + kg * D + i);
-      if (CH) gs[idx] = dr_decay<T>(A, row, h, h * D + i);
+      if (CH) gs[idx] = dr_decay<T>(A, row, rate, h * D + i);
     }
     for (int idx = tid; idx < nt * VS; idx += 256) {
       const int tt = idx / VS, jj = idx - tt * VS;
@@ -192,7 +194,7 @@ __global__ void __launch_bounds__(256) delta_rule_kernel(
           ? IO<T>::ld(A.v + row * A.v_stride + h * Dv + v0 + jj) : 0.f;
     }
     if (tid < nt)
-      dr_gates<T, CH>(A, tb + tid, h, sc + tid * DR_NS + 3,
+      dr_gates<T, CH>(A, tb + tid, h, rate, sc + tid * DR_NS + 3,
                       sc + tid * DR_NS + 4);
     __syncthreads();
     {                                     // unit scales: 16 lanes per token
@@ -426,12 +428,13 @@ __global__ void __launch_bounds__(256) delta_rule_decode_kernel(
   float* pq = pa + RG * Dv;         // [RG][Dv] partial S^T q
   float* gs = pq + RG * Dv;         // [D] channel decays (CH)
   const int rg = tid / TCn, tc = tid - rg * TCn;
+  const float rate = -expf(A.A_log[h]);
   float sq = 0.f, sk = 0.f, skq = 0.f;
   for (int i = tid; i < D; i += 256) {
     const float qv = IO<T>::ld(A.q + s * A.q_stride + kg * D + i);
     const float kv = IO<T>::ld(A.k + s * A.k_stride + kg * D + i);
     qs[i] = qv; ks[i] = kv;
-    if (CH) gs[i] = dr_decay<T>(A, s, h, h * D + i);
+    if (CH) gs[i] = dr_decay<T>(A, s, rate, h * D + i);
     sq += qv * qv; sk += kv * kv; skq += qv * kv;
   }
   for (int i = tid; i < Dv; i += 256)
@@ -450,7 +453,7 @@ __global__ void __launch_bounds__(256) delta_rule_decode_kernel(
   const float qscale = 1.0f / sqrtf((float)D) / sqrtf(sq + 1e-6f);
   const float kq = skq * kscale * qscale;
   float g, beta;
-  dr_gates<T, CH>(A, s, h, &g, &beta);
+  dr_gates<T, CH>(A, s, h, rate, &g, &beta);
   const int slot = slots[s];
   const bool load = slot >= 0 && ctx_lens[s] > 0;
   float* sp = state + (((long)max(slot, 0) * heads + h) * D) * (long)Dv + 4 * tc;

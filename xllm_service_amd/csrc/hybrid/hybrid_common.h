@@ -25,6 +25,29 @@ template <> struct IO<unsigned short> {
 XLLM_DEV float sigmoidf_(float x) { return 1.0f / (1.0f + __expf(-x)); }
 XLLM_DEV float siluf_(float x) { return x / (1.0f + __expf(-x)); }
 
+// two neighbouring values at once (8 B of fp32, 4 B of bf16)
+template <typename T> struct Pair;
+template <> struct Pair<float> {
+  static XLLM_DEV void ld(const float* p, float& a, float& b) {
+    const float2 x = *reinterpret_cast<const float2*>(p);
+    a = x.x; b = x.y;
+  }
+  static XLLM_DEV void st(float* p, float a, float b) {
+    *reinterpret_cast<float2*>(p) = make_float2(a, b);
+  }
+};
+template <> struct Pair<unsigned short> {
+  static XLLM_DEV void ld(const unsigned short* p, float& a, float& b) {
+    const unsigned x = *reinterpret_cast<const unsigned*>(p);
+    a = bf16_to_f32((unsigned short)(x & 0xffffu));
+    b = bf16_to_f32((unsigned short)(x >> 16));
+  }
+  static XLLM_DEV void st(unsigned short* p, float a, float b) {
+    *reinterpret_cast<unsigned*>(p) =
+        (unsigned)f32_to_bf16(a) | ((unsigned)f32_to_bf16(b) << 16);
+  }
+};
+
 // four neighbouring values at once (16 B of fp32, 8 B of bf16)
 template <typename T> struct Quad;
 template <> struct Quad<float> {

@@ -40,7 +40,9 @@ XLLM_DEV int seq_of_token(const int* __restrict__ cu_q, int n_seqs, int t) {
 // TAPS > 0: the filter length is a compile-time constant, the filter and a
 // sliding window of the last inputs stay in registers, and every token of the
 // tile costs one new input load. TAPS == 0: any length, every tap loaded.
-template <typename T, int TAPS>
+// VEC: heads of an even width and rows aligned to channel pairs, a pair is
+// one access.
+template <typename T, int TAPS, bool VEC>
 __global__ void __launch_bounds__(256) short_conv_kernel(
     T* __restrict__ out, long out_stride, T* __restrict__ cache,
     const long* __restrict__ slot_mapping, int block_size,
@@ -57,7 +59,7 @@ __global__ void __launch_bounds__(256) short_conv_kernel(
   const int h = idx / ppairs, j = idx - h * ppairs;
   const int d0 = 2 * j;
   const int c0 = h * hd + d0;
-  const bool two = d0 + 1 < hd;
+  const bool two = VEC || d0 + 1 < hd;
   const int K1 = taps - 1;
   const float b0 = bias ? IO<T>::ld(bias + c0) : 0.f;
   const float b1 = (bias && two) ? IO<T>::ld(bias + c0 + 1) : 0.f;
@@ -100,6 +102,7 @@ __global__ void __launch_bounds__(256) short_conv_kernel(
         if (slot < 0) return;
         row = state + ((long)slot * K1 + (K1 + src)) * state_row + state_off + c0;
       }
+      if (VEC) { Pair<T>::ld(row, u0, u1); return; }
       u0 = IO<T>::ld(row);
       if (two) u1 = IO<T>::ld(row + 1);
     };
@@ -128,8 +131,10 @@ __global__ void __launch_bounds__(256) short_conv_kernel(
       if (TAPS > 0) {
 #pragma unroll
         for (int jj = 0; jj < NT - 1; ++jj) {
-          IO<T>::st(st + (long)jj * state_row, h0[jj + 1]);
-          if (two) IO<T>::st(st + (long)jj * state_row + 1, h1[jj + 1]);
+          T* sr = st + (long)jj * state_row;
+          if (VEC) { Pair<T>::st(sr, h0[jj + 1], h1[jj + 1]); continue; }
+          IO<T>::st(sr, h0[jj + 1]);
+          if (two) IO<T>::st(sr + 1, h1[jj + 1]);
         }
       } else {
         for (int jj = 0; jj < K1; ++jj) {  // ascending: reads run ahead
@@ -151,9 +156,15 @@ __global__ void __launch_bounds__(256) short_conv_kernel(
       a1 = v * cf + u * sf;
     }
     if (add_input) {
-      const T* row = x + (long)t * x_stride + c0;
-      a0 += IO<T>::ld(row);
-      if (two) a1 += IO<T>::ld(row + 1);
+      float u0, u1 = 0.f;
+      if (TAPS > 0) {                      // the window's last entry
+        u0 = h0[NT - 1]; u1 = h1[NT - 1];
+      } else {
+        const T* row = x + (long)t * x_stride + c0;
+        u0 = IO<T>::ld(row);
+        if (two) u1 = IO<T>::ld(row + 1);
+      }
+      a0 += u0; a1 += u1;
     }
     T* dst;
     if (cache) {
@@ -164,6 +175,7 @@ __global__ void __launch_bounds__(256) short_conv_kernel(
     } else {
       dst = out + (long)t * out_stride + c0;
     }
+    if (VEC) { Pair<T>::st(dst, a0, a1); continue; }
     IO<T>::st(dst, a0);
     if (two) IO<T>::st(dst + 1, a1);
   }
@@ -210,8 +222,23 @@ void launch_short_conv(T* out, long out_stride, T* cache,
   // short ones (decode) keep every token in a workgroup of its own
   const int tile = tokens >= 2048 ? 16 : tokens >= 256 ? 4 : 1;
   dim3 grid((n + bx - 1) / bx, (tokens + tile - 1) / tile);
+  // every row a thread touches starts on a channel pair
+  auto even = [](const void* p, long stride) {
+    return reinterpret_cast<uintptr_t>(p) % (2 * sizeof(T)) == 0 &&
+           stride % 2 == 0;
+  };
+  const bool vec = hd % 2 == 0 && even(x, x_stride) &&
+                   (taps == 1 || even(state, state_row)) &&
+                   state_off % 2 == 0 && even(out, out_stride) &&
+                   even(cache, 0);
 #define SC_LAUNCH(TAPS)                                                       \
-  hipLaunchKernelGGL((short_conv_kernel<T, TAPS>), grid, dim3(bx), 0, st, out, \
+  do {                                                                        \
+    if (vec) SC_LAUNCH_AS(TAPS, true);                                        \
+    else SC_LAUNCH_AS(TAPS, false);                                           \
+  } while (0)
+#define SC_LAUNCH_AS(TAPS, VEC)                                               \
+  hipLaunchKernelGGL((short_conv_kernel<T, TAPS, VEC>), grid, dim3(bx), 0,    \
+                     st, out,                                                 \
                      out_stride, cache, slot_mapping, block_size, x, x_stride, \
                      w, bias, state, state_row, state_off, slots, cu_q,       \
                      ctx_lens, n_seqs, heads, hd, taps, act_silu, rot_dims,   \
@@ -223,6 +250,7 @@ void launch_short_conv(T* out, long out_stride, T* cache,
     default: SC_LAUNCH(0); break;
   }
 #undef SC_LAUNCH
+#undef SC_LAUNCH_AS
 }
 
 template <typename T>
