@@ -63,7 +63,7 @@ def _variants():
             parallel(heads=6, kv_heads=2, dim=64, vdim=40, dims=48, size=33,
                      base=1e4, s_heads=4, s_vdim=32, state=24,
                      mlp=moe(ff=48, experts=7, top=2)),
-            latent(heads=6, dim=32, rot_dim=16, vdim=24, rank=80, size=40,
+            latent(heads=6, dim=32, rot_dim=16, vdim=24, rank=80, size=36,
                    base=1e3, mlp=dense(192, 2.0)),
             delta(heads=4, kv_heads=2, dim=48, vdim=32, conv=4,
                   mlp=dense(96)),

@@ -97,7 +97,7 @@ def test_depth_average_with_two_norms(target, W, f32):
 
 
 @pytest.mark.parametrize("target", TARGETS)
-@pytest.mark.parametrize("F", [5, 12, 320])
+@pytest.mark.parametrize("F", [5, 12, 352])
 @pytest.mark.parametrize("limit", [0.5, 7.0])
 def test_clamped_gate(target, F, limit):
     """The gate has no lower bound, the up half has both."""
@@ -369,7 +369,7 @@ def _latent_case(target, H, r, rd, L, asked, window, standout, seed,
 
 @pytest.mark.parametrize("target", TARGETS)
 @pytest.mark.parametrize("decode", [False, True])
-@pytest.mark.parametrize("H,r,rd", [(2, 9, 4), (4, 96, 32), (20, 64, 16),
+@pytest.mark.parametrize("H,r,rd", [(2, 9, 4), (4, 88, 24), (20, 64, 16),
                                     (3, 200, 40), (2, 512, 64), (40, 40, 8)])
 def test_latent_window_edges(target, decode, H, r, rd):
     L, window = 150, 37
