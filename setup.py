@@ -47,7 +47,7 @@ ext_modules = [
         },
     ),
     # hybrid sequence mixers (latent attention, decayed and gated linear
-    # recurrences, the gated delta rule, soft-capped / windowed paged attention,
+    # recurrences, the gated delta rule, retention, soft-capped / windowed paged attention,
     # short convolutions, rotary turns with head norms), grouped and post
     # norms, PolyNorm, residual streams, depth averages and routed experts;
     # bf16 and fp32 activations
@@ -60,7 +60,8 @@ ext_modules = [
                       "streams.hip", "short_conv.hip",
                       "gated_recurrence.hip", "capped_attn.hip",
                       "capped_attn_mfma.hip", "rownorm_rope.hip",
-                      "delta_rule.hip", "rope_headnorm.hip", "depth_mix.hip")
+                      "delta_rule.hip", "rope_headnorm.hip", "depth_mix.hip",
+                      "retention.hip", "joint_layer.hip")
         ],
         extra_compile_args={
             "cxx": ["-O3", "-std=c++17"],

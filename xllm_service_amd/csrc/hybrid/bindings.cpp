@@ -29,7 +29,8 @@ template <typename T>
 void launch_rope_headnorm_store(T*, const T*, const T*, const T*, long, long,
                                 long, const long*, const double*, int, int,
                                 int, float, int, int, int, int, int, T*, T*,
-                                const long*, int, float, hipStream_t);
+                                const long*, int, float, const float*,
+                                const float*, const float*, hipStream_t);
 template <typename T>
 void launch_polynorm(T*, const T*, const float*, float, long, int, long,
                      hipStream_t);
@@ -74,7 +75,7 @@ void launch_decay_attn(float*, const T*, const T*, const T*, const float*,
                        int, int, long, long, long, int, int, float*,
                        hipStream_t);
 void launch_moe_route(int*, float*, const float*, int, int, int, int, int,
-                      int, const float*, int, int, hipStream_t);
+                      int, const float*, int, int, float, hipStream_t);
 template <typename T>
 void launch_moe_combine(float*, const T*, const int*, const float*, long, int,
                         int, const T*, long, const T*, long, hipStream_t);
@@ -111,16 +112,16 @@ void launch_gated_recurrence(int, float*, const T*, const T*, const T*,
 template <typename T>
 void launch_gated_group_norm(T*, const float*, const float*, int, const T*,
                              long, float, int, int, int, int, int,
-                             hipStream_t);
+                             long, hipStream_t);
 int capped_attn_mfma_class(int D, int Dv);
-void launch_capped_attn_mfma(float*, float*, float*, const unsigned short*,
+void launch_capped_attn_mfma(void*, long, int, float*, float*, const unsigned short*,
                              const unsigned short*, const unsigned short*,
                              const int*, const int*, const int*, int, int, int,
                              int, int, int, int, int, float, float, long, int,
                              int, const float*, int, const float*, int,
                              hipStream_t);
-template <typename T>
-void launch_capped_attn(float*, const T*, const T*, const T*, const int*,
+template <typename T, typename TO>
+void launch_capped_attn(TO*, long, const T*, const T*, const T*, const int*,
                         const int*, const int*, int, int, int, int, int, int,
                         int, int, float, float, long, int, const float*, int,
                         const float*, int, hipStream_t);
@@ -136,6 +137,23 @@ void launch_clamped_glu(T*, const T*, long, int, float, float, float,
 template <typename T>
 void launch_gelu_scaled(T*, const T*, long, int, const float*, const int*,
                         const float*, int, int, hipStream_t);
+template <typename T>
+void launch_join_norm(float*, T*, int, const T*, long, const long*, float,
+                      const T*, const int*, const float*, int, const float*,
+                      float, long, int, hipStream_t);
+template <typename T>
+void launch_glu_rows(T*, long, const T*, long, const T*, long, const T*, long,
+                     long, int, int, hipStream_t);
+void launch_rope_table(float*, const long*, const double*, int, int, float,
+                       hipStream_t);
+long retention_chunks(long, long);
+int retention_fused_columns();
+template <typename T>
+void launch_retention(T*, long, float*, const T*, long, float, float*,
+                      const T*, const T*, const T*, long, long, long,
+                      const float*, int, float, const float*, float*,
+                      const int*, const int*, const int*, long, int, int, int,
+                      int, hipStream_t);
 }  // namespace hyb
 }  // namespace xllm
 
@@ -284,24 +302,27 @@ void gelu_tanh_gate(Tensor out, Tensor g, Tensor u) {
 }
 
 // q_out [T, H*D] contiguous; q/k/v row views of a projection (v absent: the
-// values are the keys); caches [blocks, n_kv, block, D | Dv]
-void rope_headnorm_store(Tensor q_out, Tensor q, Tensor k,
+// values are the keys, or k is absent too: queries only); caches [blocks, n_kv,
+// block, D | Dv]; q_w/k_w fp32 [D]: head norm before the turn; table fp32
+// [T, rot]: cos | sin per token
+void rope_headnorm_store(Tensor q_out, Tensor q, c10::optional<Tensor> k,
                          c10::optional<Tensor> v, Tensor pos, Tensor inv_freq,
                          long rot, bool pairs, bool unit, double eps,
                          long heads, long n_kv, Tensor k_cache,
-                         Tensor v_cache, Tensor slot_mapping, double mscale) {
-  CHK_ACT(q_out); CHK_ACT(q); CHK_ACT(k); CHK_I64C(pos);
+                         Tensor v_cache, Tensor slot_mapping, double mscale,
+                         c10::optional<Tensor> q_w, c10::optional<Tensor> k_w,
+                         c10::optional<Tensor> table) {
+  CHK_ACT(q_out); CHK_ACT(q); CHK_I64C(pos);
   CHK_I64C(slot_mapping); CHK_ACT(k_cache); CHK_ACT(v_cache);
-  TORCH_CHECK(q.dim() == 2 && k.dim() == 2 && q_out.is_contiguous() &&
+  TORCH_CHECK(q.dim() == 2 && q_out.is_contiguous() &&
               k_cache.dim() == 4 && v_cache.dim() == 4 &&
               k_cache.is_contiguous() && v_cache.is_contiguous());
-  TORCH_CHECK(q.dtype() == k.dtype() && q.dtype() == q_out.dtype() &&
+  TORCH_CHECK(q.dtype() == q_out.dtype() &&
               q.dtype() == k_cache.dtype() && q.dtype() == v_cache.dtype());
   const int T = q.size(0), D = k_cache.size(3), Dv = v_cache.size(3);
   const int bs = k_cache.size(2);
   TORCH_CHECK(heads >= 1 && n_kv >= 1 && D <= 64 * 8 &&
-              q.size(1) == heads * D && k.size(1) == n_kv * D &&
-              k.size(0) == T && q_out.numel() == q.numel() &&
+              q.size(1) == heads * D && q_out.numel() == q.numel() &&
               k_cache.size(1) == n_kv && v_cache.size(1) == n_kv &&
               v_cache.size(2) == bs && v_cache.size(0) == k_cache.size(0) &&
               pos.numel() == T && slot_mapping.numel() == T,
@@ -309,20 +330,40 @@ void rope_headnorm_store(Tensor q_out, Tensor q, Tensor k,
   TORCH_CHECK(rot >= 0 && rot % 2 == 0 && rot <= D &&
               inv_freq.is_cuda() && inv_freq.dtype() == torch::kDouble &&
               inv_freq.is_contiguous() && inv_freq.numel() == rot / 2);
-  const void* vp = nullptr;
-  long vs = 0;
+  const void *kp = nullptr, *vp = nullptr;
+  long ks = 0, vs = 0;
+  if (k.has_value()) {
+    CHK_ACT(*k);
+    TORCH_CHECK(k->dim() == 2 && k->dtype() == q.dtype() &&
+                k->size(0) == T && k->size(1) == n_kv * D,
+                "rope_headnorm_store: bad key rows");
+    kp = k->data_ptr();
+    ks = k->stride(0);
+  }
   if (v.has_value()) {
     CHK_ACT(*v);
-    TORCH_CHECK(v->dim() == 2 && v->dtype() == q.dtype() &&
+    TORCH_CHECK(kp != nullptr && v->dim() == 2 && v->dtype() == q.dtype() &&
                 v->size(0) == T && v->size(1) == n_kv * Dv,
                 "rope_headnorm_store: bad value rows");
     vp = v->data_ptr();
     vs = v->stride(0);
   }
-  if (is_f32(q))
-    hy::launch_rope_headnorm_store<float>(ptr<float>(q_out), ptr<float>(q), ptr<float>(k), (const float*)vp, q.stride(0), k.stride(0), vs, ptr<long>(pos), ptr<double>(inv_freq), rot, pairs, unit, eps, T, heads, n_kv, D, Dv, ptr<float>(k_cache), ptr<float>(v_cache), ptr<long>(slot_mapping), bs, mscale, cur());
-  else
-    hy::launch_rope_headnorm_store<bf>(ptr<bf>(q_out), ptr<bf>(q), ptr<bf>(k), (const bf*)vp, q.stride(0), k.stride(0), vs, ptr<long>(pos), ptr<double>(inv_freq), rot, pairs, unit, eps, T, heads, n_kv, D, Dv, ptr<bf>(k_cache), ptr<bf>(v_cache), ptr<long>(slot_mapping), bs, mscale, cur());
+  auto f32 = [&](const c10::optional<Tensor>& t, long n) -> const float* {
+    if (!t.has_value()) return nullptr;
+    CHK_F32C(*t);
+    TORCH_CHECK(t->numel() == n, "rope_headnorm_store: bad fp32 operand");
+    return ptr<float>(*t);
+  };
+  const float *wq = f32(q_w, D), *wk = f32(k_w, D);
+  const float* tp = rot ? f32(table, (long)T * rot) : nullptr;
+#define RHS_CALL(T_)                                                          \
+  hy::launch_rope_headnorm_store<T_>(                                         \
+      ptr<T_>(q_out), ptr<T_>(q), (const T_*)kp, (const T_*)vp, q.stride(0),  \
+      ks, vs, ptr<long>(pos), ptr<double>(inv_freq), rot, pairs, unit, eps, T,\
+      heads, n_kv, D, Dv, ptr<T_>(k_cache), ptr<T_>(v_cache),                 \
+      ptr<long>(slot_mapping), bs, mscale, wq, wk, tp, cur())
+  if (is_f32(q)) RHS_CALL(float); else RHS_CALL(bf);
+#undef RHS_CALL
 }
 
 void gelu_tanh_mul(Tensor out, Tensor x) {
@@ -602,7 +643,7 @@ void decay_attn(Tensor out, Tensor q, Tensor k, Tensor v, Tensor decay,
 // z fp32 [T, E] router logits -> ids int32 [T, top], wts fp32 [T, top]
 void moe_route(Tensor ids, Tensor wts, Tensor z, long top, long n_groups,
                long keep, bool softmax, c10::optional<Tensor> correction,
-               bool group_max, bool normalize) {
+               bool group_max, bool normalize, double scale) {
   CHK_I32C(ids); CHK_F32C(wts); CHK_F32C(z);
   TORCH_CHECK(z.dim() == 2);
   const int T = z.size(0), E = z.size(1);
@@ -619,7 +660,7 @@ void moe_route(Tensor ids, Tensor wts, Tensor z, long top, long n_groups,
   }
   hy::launch_moe_route(ptr<int>(ids), ptr<float>(wts), ptr<float>(z), T, E,
                        top, n_groups, keep, softmax, corr, group_max,
-                       normalize, cur());
+                       normalize, scale, cur());
 }
 
 // out fp32 [T, width]; y [R, width] contiguous; rows int32 [T, top] < R; wts
@@ -946,30 +987,39 @@ void gated_recurrence(long kind, Tensor out, Tensor q, Tensor k, Tensor v,
     hy::launch_gated_recurrence<bf>(kind, ptr<float>(out), ptr<bf>(q), ptr<bf>(k), ptr<bf>(v), ptr<bf>(g), q.stride(0), k.stride(0), v.stride(0), g.stride(0), ptr<float>(p0), p1p, p2p, c0, c1, ptr<float>(state), ptr<int>(slots), cu, ptr<int>(ctx_lens), n_seqs, H, groups, D, Dv, chunk, max_chunks, wsp, wap, cur());
 }
 
-// out [rows, n] from o fp32 [rows, n], gate [rows, n] (row view), w fp32 with
-// n or n/groups entries
-void gated_group_norm(Tensor out, Tensor o, Tensor w, Tensor gate, double eps,
-                      long groups, bool act_silu, bool gate_first) {
-  CHK_ACT(out); CHK_F32C(o); CHK_F32C(w); CHK_ACT(gate);
-  TORCH_CHECK(out.is_contiguous() && out.dim() == 2 && gate.dim() == 2);
+// out [rows, n] (row view) from o fp32 [rows, n], gate [rows, n] (row view), w
+// fp32 with n or n/groups entries (absent: no weight)
+void gated_group_norm(Tensor out, Tensor o, c10::optional<Tensor> w,
+                      Tensor gate, double eps, long groups, bool act_silu,
+                      bool gate_first) {
+  CHK_ACT(out); CHK_F32C(o); CHK_ACT(gate);
+  TORCH_CHECK(out.dim() == 2 && gate.dim() == 2);
   const int rows = out.size(0), n = out.size(1);
   TORCH_CHECK(o.numel() == (long)rows * n && gate.size(0) == rows &&
               gate.size(1) == n && gate.dtype() == out.dtype() &&
-              groups >= 1 && n % groups == 0 &&
-              (w.numel() == n || w.numel() == n / groups));
+              groups >= 1 && n % groups == 0);
+  const float* wp = nullptr;
+  int period = n;
+  if (w.has_value()) {
+    CHK_F32C(*w);
+    period = w->numel();
+    TORCH_CHECK(period == n || period == n / groups);
+    wp = ptr<float>(*w);
+  }
   if (is_f32(out))
-    hy::launch_gated_group_norm<float>(ptr<float>(out), ptr<float>(o), ptr<float>(w), w.numel(), ptr<float>(gate), gate.stride(0), eps, rows, n, groups, act_silu, gate_first, cur());
+    hy::launch_gated_group_norm<float>(ptr<float>(out), ptr<float>(o), wp, period, ptr<float>(gate), gate.stride(0), eps, rows, n, groups, act_silu, gate_first, out.stride(0), cur());
   else
-    hy::launch_gated_group_norm<bf>(ptr<bf>(out), ptr<float>(o), ptr<float>(w), w.numel(), ptr<bf>(gate), gate.stride(0), eps, rows, n, groups, act_silu, gate_first, cur());
+    hy::launch_gated_group_norm<bf>(ptr<bf>(out), ptr<float>(o), wp, period, ptr<bf>(gate), gate.stride(0), eps, rows, n, groups, act_silu, gate_first, out.stride(0), cur());
 }
 
-// out fp32 [T, H, Dv]; q [T, H*D] row view; caches [blocks, n_kv, bs, D|Dv]
+// out: fp32 [T, H, Dv] contiguous, or [T, H*Dv] rows (a view with a stride) of
+// fp32 or q's type; q [T, H*D] row view; caches [blocks, n_kv, bs, D|Dv]
 void capped_attn(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
                  Tensor block_tables, c10::optional<Tensor> cu_q,
                  Tensor seq_lens, long heads, double scale, double cap,
                  long window, c10::optional<Tensor> sink, long keep_first,
                  c10::optional<Tensor> head_scale, bool chunked) {
-  CHK_F32C(out); CHK_ACT(q); CHK_ACT(k_cache); CHK_ACT(v_cache);
+  CHK_ACT(out); CHK_ACT(q); CHK_ACT(k_cache); CHK_ACT(v_cache);
   CHK_I32C(block_tables); CHK_I32C(seq_lens);
   TORCH_CHECK(q.dim() == 2 && k_cache.dim() == 4 && v_cache.dim() == 4 &&
               k_cache.is_contiguous() && v_cache.is_contiguous() &&
@@ -981,7 +1031,12 @@ void capped_attn(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
               v_cache.size(1) == n_kv && v_cache.size(2) == bs &&
               v_cache.size(0) == k_cache.size(0) && Dv <= 64 * 8,
               "capped_attn: bad shapes");
-  TORCH_CHECK(out.numel() == (long)T * heads * Dv);
+  TORCH_CHECK(out.numel() == (long)T * heads * Dv &&
+              (is_f32(out) || out.dtype() == q.dtype()) &&
+              (out.is_contiguous() || out.dim() == 2),
+              "capped_attn: bad output");
+  const long out_stride = out.dim() == 2 ? out.stride(0) : (long)heads * Dv;
+  const bool out_bf = is_bf16(out);
   const int n_seqs = seq_lens.numel();
   TORCH_CHECK(block_tables.size(0) == n_seqs);
   const int* cu = nullptr;
@@ -1010,7 +1065,9 @@ void capped_attn(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
   // bf16: MFMA kernel when the sizes fit one of its instantiations
   if (is_bf16(q) && hy::capped_attn_mfma_class(D, Dv) != 0 &&
       q.stride(0) % 8 == 0 &&
-      reinterpret_cast<uintptr_t>(q.data_ptr()) % 16 == 0) {
+      reinterpret_cast<uintptr_t>(q.data_ptr()) % 16 == 0 &&
+      out_stride % 4 == 0 &&
+      reinterpret_cast<uintptr_t>(out.data_ptr()) % (out_bf ? 8 : 16) == 0) {
     int n_part = 1;
     Tensor ws_acc, ws_ml;
     if (cu == nullptr) {
@@ -1033,11 +1090,12 @@ void capped_attn(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
         n_part = std::min(32, std::max(1, std::atoi(e)));
     }
     if (n_part > 1) {
-      ws_acc = torch::empty({(long)T * heads * n_part, (long)Dv}, out.options());
-      ws_ml = torch::empty({(long)T * heads * n_part, 2}, out.options());
+      const auto f32 = out.options().dtype(torch::kFloat);
+      ws_acc = torch::empty({(long)T * heads * n_part, (long)Dv}, f32);
+      ws_ml = torch::empty({(long)T * heads * n_part, 2}, f32);
     }
     hy::launch_capped_attn_mfma(
-        ptr<float>(out), n_part > 1 ? ptr<float>(ws_acc) : nullptr,
+        out.data_ptr(), out_stride, out_bf, n_part > 1 ? ptr<float>(ws_acc) : nullptr,
         n_part > 1 ? ptr<float>(ws_ml) : nullptr, ptr<bf>(q), ptr<bf>(k_cache),
         ptr<bf>(v_cache), ptr<int>(block_tables), cu, ptr<int>(seq_lens), T,
         n_seqs, heads, n_kv, D, Dv, bs, block_tables.size(1), scale, cap,
@@ -1045,10 +1103,16 @@ void capped_attn(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
     return;
   }
   TORCH_CHECK((size_t)4 * D * 4 <= 64 * 1024, "query row too wide for LDS");
-  if (is_f32(q))
-    hy::launch_capped_attn<float>(ptr<float>(out), ptr<float>(q), ptr<float>(k_cache), ptr<float>(v_cache), ptr<int>(block_tables), cu, ptr<int>(seq_lens), T, n_seqs, heads, n_kv, D, Dv, bs, block_tables.size(1), scale, cap, q.stride(0), window, sinkp, keep_first, hsp, chunked, cur());
-  else
-    hy::launch_capped_attn<bf>(ptr<float>(out), ptr<bf>(q), ptr<bf>(k_cache), ptr<bf>(v_cache), ptr<int>(block_tables), cu, ptr<int>(seq_lens), T, n_seqs, heads, n_kv, D, Dv, bs, block_tables.size(1), scale, cap, q.stride(0), window, sinkp, keep_first, hsp, chunked, cur());
+#define CA_CALL(T_, TO_)                                                      \
+  hy::launch_capped_attn<T_, TO_>(                                            \
+      ptr<TO_>(out), out_stride, ptr<T_>(q), ptr<T_>(k_cache),                \
+      ptr<T_>(v_cache), ptr<int>(block_tables), cu, ptr<int>(seq_lens), T,    \
+      n_seqs, heads, n_kv, D, Dv, bs, block_tables.size(1), scale, cap,       \
+      q.stride(0), window, sinkp, keep_first, hsp, chunked, cur())
+  if (is_f32(q)) CA_CALL(float, float);
+  else if (out_bf) CA_CALL(bf, bf);
+  else CA_CALL(bf, float);
+#undef CA_CALL
 }
 
 // One layer's result and what follows it, see depth_mix.hip. h1 (h2) [T, W]
@@ -1157,6 +1221,137 @@ void gelu_scaled(Tensor out, Tensor x, c10::optional<Tensor> scale,
   else hy::launch_gelu_scaled<bf>(ptr<bf>(out), ptr<bf>(x), rows, F, sp, ip, wp, tokens, top, cur());
 }
 
+// x fp32 [T, W] in place (written only with `fresh`); h [T, W] contiguous; y
+// [T, W] row view of h's type, or with ids int64 [T] a table [V, W]; e [R, W]
+// of that type with rows int32 [T, top] < R and wts fp32 [T, top]; w fp32 [W]
+void join_norm(Tensor x, Tensor h, bool fresh, Tensor y,
+               c10::optional<Tensor> ids, double a, c10::optional<Tensor> e,
+               c10::optional<Tensor> rows, c10::optional<Tensor> wts, Tensor w,
+               double eps) {
+  CHK_F32C(x); CHK_ACT(h); CHK_ACT(y); CHK_F32C(w);
+  TORCH_CHECK(x.dim() == 2 && h.dim() == 2 && y.dim() == 2 &&
+              h.is_contiguous() && y.dtype() == h.dtype());
+  const long T = x.size(0);
+  const int W = x.size(1);
+  TORCH_CHECK(h.size(0) == T && h.size(1) == W && y.size(1) == W &&
+              w.numel() == W, "join_norm: bad shapes");
+  TORCH_CHECK((size_t)W * 4 <= 60 * 1024, "width too large for LDS");
+  const long* ip = nullptr;
+  if (ids.has_value()) {
+    CHK_I64C(*ids);
+    TORCH_CHECK(ids->numel() == T);
+    ip = ptr<long>(*ids);
+  } else {
+    TORCH_CHECK(y.size(0) == T);
+  }
+  const void* ep = nullptr;
+  const int* rp = nullptr;
+  const float* wp = nullptr;
+  int top = 0;
+  if (e.has_value()) {
+    TORCH_CHECK(rows.has_value() && wts.has_value());
+    CHK_ACT(*e); CHK_I32C(*rows); CHK_F32C(*wts);
+    TORCH_CHECK(e->is_contiguous() && e->size(-1) == W &&
+                e->dtype() == h.dtype() && rows->dim() == 2 &&
+                rows->size(0) == T && wts->numel() == rows->numel(),
+                "join_norm: bad expert rows");
+    ep = e->data_ptr();
+    rp = ptr<int>(*rows);
+    wp = ptr<float>(*wts);
+    top = rows->size(1);
+  }
+  if (is_f32(h))
+    hy::launch_join_norm<float>(ptr<float>(x), ptr<float>(h), fresh, ptr<float>(y), y.stride(0), ip, a, (const float*)ep, rp, wp, top, ptr<float>(w), eps, T, W, cur());
+  else
+    hy::launch_join_norm<bf>(ptr<float>(x), ptr<bf>(h), fresh, ptr<bf>(y), y.stride(0), ip, a, (const bf*)ep, rp, wp, top, ptr<float>(w), eps, T, W, cur());
+}
+
+// out, g, u [rows, F] row views of one type; s [rows, 1] of that type
+void glu_rows(Tensor out, Tensor g, Tensor u, c10::optional<Tensor> s,
+              bool gelu) {
+  CHK_ACT(out); CHK_ACT(g); CHK_ACT(u);
+  TORCH_CHECK(out.dim() == 2 && g.sizes() == out.sizes() &&
+              u.sizes() == out.sizes() && g.dtype() == out.dtype() &&
+              u.dtype() == out.dtype(), "glu_rows: bad shapes");
+  const void* sp = nullptr;
+  long ss = 0;
+  if (s.has_value()) {
+    TORCH_CHECK(s->is_cuda() && s->dtype() == out.dtype() && s->dim() == 2 &&
+                s->size(0) == out.size(0) && s->size(1) == 1);
+    sp = s->data_ptr();
+    ss = s->stride(0);
+  }
+  if (is_f32(out))
+    hy::launch_glu_rows<float>(ptr<float>(out), out.stride(0), ptr<float>(g), g.stride(0), ptr<float>(u), u.stride(0), (const float*)sp, ss, out.size(0), out.size(1), gelu, cur());
+  else
+    hy::launch_glu_rows<bf>(ptr<bf>(out), out.stride(0), ptr<bf>(g), g.stride(0), ptr<bf>(u), u.stride(0), (const bf*)sp, ss, out.size(0), out.size(1), gelu, cur());
+}
+
+// table fp32 [T, 2 * n]: cos | sin of pos * inv_freq (fp64 [n])
+void rope_table(Tensor table, Tensor pos, Tensor inv_freq, double mscale) {
+  CHK_F32C(table); CHK_I64C(pos);
+  TORCH_CHECK(inv_freq.is_cuda() && inv_freq.dtype() == torch::kDouble &&
+              inv_freq.is_contiguous());
+  const long T = pos.numel(), n = inv_freq.numel();
+  TORCH_CHECK(table.numel() == T * 2 * n, "rope_table: bad shapes");
+  hy::launch_rope_table(ptr<float>(table), ptr<long>(pos),
+                        ptr<double>(inv_freq), T, n, mscale, cur());
+}
+
+// out, gate [T, H*Dv], q, k [T, H*D], v [T, H*Dv] row views of one type; table
+// fp32 [T, rot]; state fp32 [slots, H, D, Dv]; cu_q absent: one token per
+// sequence
+void retention(Tensor out, Tensor q, Tensor k, Tensor v, Tensor gate,
+               Tensor table, double k_scale, Tensor decay, Tensor state,
+               Tensor slots, c10::optional<Tensor> cu_q, Tensor ctx_lens,
+               double eps) {
+  CHK_ACT(out); CHK_ACT(q); CHK_ACT(k); CHK_ACT(v); CHK_ACT(gate);
+  CHK_F32C(table); CHK_F32C(decay); CHK_F32C(state); CHK_I32C(slots);
+  CHK_I32C(ctx_lens);
+  TORCH_CHECK(state.dim() == 4 && q.dim() == 2 && k.dim() == 2 &&
+              v.dim() == 2 && gate.dim() == 2 && out.dim() == 2 &&
+              table.dim() == 2 && q.dtype() == k.dtype() &&
+              q.dtype() == v.dtype() && q.dtype() == gate.dtype() &&
+              q.dtype() == out.dtype());
+  const int H = state.size(1), D = state.size(2), Dv = state.size(3);
+  const long T = q.size(0);
+  const int rot = table.size(1);
+  TORCH_CHECK(q.size(1) == H * D && k.size(1) == H * D && v.size(1) == H * Dv &&
+              gate.size(1) == H * Dv && out.size(1) == H * Dv &&
+              k.size(0) == T && v.size(0) == T && gate.size(0) == T &&
+              out.size(0) == T && table.size(0) == T && decay.numel() == H &&
+              rot % 2 == 0 && rot <= D, "retention: bad shapes");
+  TORCH_CHECK(D <= 256, "key width > 256 unsupported");
+  const int n_seqs = slots.numel();
+  TORCH_CHECK(ctx_lens.numel() == n_seqs);
+  const int* cu = nullptr;
+  Tensor ws, raw;
+  if (cu_q.has_value()) {
+    CHK_I32C(*cu_q);
+    TORCH_CHECK(cu_q->numel() == n_seqs + 1);
+    cu = ptr<int>(*cu_q);
+    ws = torch::empty({hy::retention_chunks(T, n_seqs), (long)H, (long)D,
+                       (long)Dv}, state.options());
+    if (Dv > hy::retention_fused_columns())
+      raw = torch::empty({T, (long)H * Dv}, state.options());
+  } else {
+    TORCH_CHECK(n_seqs == T, "decode: one sequence per token");
+    TORCH_CHECK(Dv <= (Dv % 4 == 0 ? 1024 : 256), "value width unsupported");
+  }
+  float* wsp = cu ? ptr<float>(ws) : nullptr;
+  float* rawp = raw.defined() ? ptr<float>(raw) : nullptr;
+#define RT_CALL(T_)                                                           \
+  hy::launch_retention<T_>(                                                   \
+      ptr<T_>(out), out.stride(0), rawp, ptr<T_>(gate), gate.stride(0), eps,  \
+      wsp, ptr<T_>(q), ptr<T_>(k), ptr<T_>(v), q.stride(0), k.stride(0),      \
+      v.stride(0), ptr<float>(table), rot, k_scale, ptr<float>(decay),        \
+      ptr<float>(state), ptr<int>(slots), cu, ptr<int>(ctx_lens), T, n_seqs,  \
+      H, D, Dv, cur())
+  if (is_f32(q)) RT_CALL(float); else RT_CALL(bf);
+#undef RT_CALL
+  if (raw.defined()) gated_group_norm(out, raw, c10::nullopt, gate, eps, H,
+                                      true, false);
+}
 }  // namespace
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
@@ -1190,4 +1385,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("depth_mix_norm", &depth_mix_norm);
   m.def("clamped_glu", &clamped_glu);
   m.def("gelu_scaled", &gelu_scaled);
+  m.def("join_norm", &join_norm);
+  m.def("glu_rows", &glu_rows);
+  m.def("rope_table", &rope_table);
+  m.def("retention", &retention);
 }

@@ -22,12 +22,12 @@ namespace hyb {
 
 constexpr int CA_MAX_ACC = 8;   // Dv <= 64 * 8
 
-// q [T, H, D] (row stride given), out fp32 [T, H, Dv].
+// q [T, H, D], out [T, H, Dv] (fp32 or the activation type), row strides given.
 // cu_q == nullptr: decode (token t is sequence t, sees seq_lens[t] keys);
 // else token t of sequence s sees seq_lens[s] - (cu_q[s+1] - 1 - t) keys.
-template <typename T>
+template <typename T, typename TO>
 __global__ void capped_attn_kernel(
-    float* __restrict__ out, const T* __restrict__ q,
+    TO* __restrict__ out, long out_stride, const T* __restrict__ q,
     const T* __restrict__ k_cache, const T* __restrict__ v_cache,
     const int* __restrict__ block_tables, const int* __restrict__ cu_q,
     const int* __restrict__ seq_lens, int n_seqs, int heads, int n_kv, int D,
@@ -123,16 +123,16 @@ __global__ void capped_attn_kernel(
     for (int i = 0; i < CA_MAX_ACC; ++i) acc[i] *= alpha;
   }
   const float inv = (l > 0.f) ? 1.0f / l : 0.f;
-  float* orow = out + ((long)t * heads + h) * Dv;
+  TO* orow = out + (long)t * out_stride + (long)h * Dv;
 #pragma unroll
   for (int i = 0; i < CA_MAX_ACC; ++i) {
     const int c = lane + 64 * i;
-    if (i < n_acc && c < Dv) orow[c] = acc[i] * inv;
+    if (i < n_acc && c < Dv) IO<TO>::st(orow + c, acc[i] * inv);
   }
 }
 
-template <typename T>
-void launch_capped_attn(float* out, const T* q, const T* k_cache,
+template <typename T, typename TO>
+void launch_capped_attn(TO* out, long out_stride, const T* q, const T* k_cache,
                         const T* v_cache, const int* block_tables,
                         const int* cu_q, const int* seq_lens, int tokens,
                         int n_seqs, int heads, int n_kv, int D, int Dv,
@@ -144,21 +144,22 @@ void launch_capped_attn(float* out, const T* q, const T* k_cache,
   if (tokens == 0) return;
   const int nw = heads < 4 ? heads : 4;
   dim3 grid(tokens, (heads + nw - 1) / nw);
-  hipLaunchKernelGGL((capped_attn_kernel<T>), grid, dim3(64 * nw),
-                     (size_t)nw * D * sizeof(float), st, out, q, k_cache,
-                     v_cache, block_tables, cu_q, seq_lens, n_seqs, heads,
+  hipLaunchKernelGGL((capped_attn_kernel<T, TO>), grid, dim3(64 * nw),
+                     (size_t)nw * D * sizeof(float), st, out, out_stride, q,
+                     k_cache, v_cache, block_tables, cu_q, seq_lens, n_seqs, heads,
                      n_kv, D, Dv, block_size, table_width, scale, cap,
                      q_row_stride, window, sink, keep_first, head_scale,
                      chunked);
 }
 
-#define INST_CA(T)                                                          \
-  template void launch_capped_attn<T>(                                      \
-      float*, const T*, const T*, const T*, const int*, const int*,         \
+#define INST_CA(T, TO)                                                      \
+  template void launch_capped_attn<T, TO>(                                  \
+      TO*, long, const T*, const T*, const T*, const int*, const int*,      \
       const int*, int, int, int, int, int, int, int, int, float, float,     \
       long, int, const float*, int, const float*, int, hipStream_t);
-INST_CA(float)
-INST_CA(unsigned short)
+INST_CA(float, float)
+INST_CA(unsigned short, float)
+INST_CA(unsigned short, unsigned short)
 
 }  // namespace hyb
 }  // namespace xllm

@@ -80,7 +80,8 @@ template <int KQ, int NO, int CS>
 __global__ void
 __launch_bounds__(256, (KQ == 4 && NO == 8 && CS == 4) ? 4 : 0)
 capped_attn_mfma_kernel(
-    float* __restrict__ out, float* __restrict__ ws_acc,
+    void* __restrict__ out, long out_stride, int out_bf16,
+    float* __restrict__ ws_acc,
     float* __restrict__ ws_ml, const unsigned short* __restrict__ q,
     const unsigned short* __restrict__ k_cache,
     const unsigned short* __restrict__ v_cache,
@@ -349,25 +350,33 @@ capped_attn_mfma_kernel(
   if (n_part == 1 && sink != nullptr) l += __expf(sink[head] - m);
   const float inv = l > 0.f ? 1.0f / l : 0.f;
   const long base = grow * n_part + blockIdx.y;
-  float* orow = (n_part == 1) ? out + grow * Dv : ws_acc + base * Dv;
   const float mul = (n_part == 1) ? inv : 1.0f;
+  const long orow = tok * out_stride + (long)head * Dv;
+  float* of = (n_part == 1) ? (float*)out + orow : ws_acc + base * Dv;
+  unsigned short* oh = (unsigned short*)out + orow;
+  const bool half_out = n_part == 1 && out_bf16;
+  // Dv % 8 == 0: a lane's four neighbouring columns are in or out together
 #pragma unroll
   for (int lb = 0; lb < NBL; ++lb)
 #pragma unroll
-    for (int nn = 0; nn < 4; ++nn)
+    for (int nn = 0; nn < 4; ++nn) {
+      const int col = ((lb * CS + cpart) * 4 + nn) * 16 + g * 4;
+      if (col >= Dv) continue;
+      float v[4];
 #pragma unroll
-      for (int rr = 0; rr < 4; ++rr) {
-        const int col = ((lb * CS + cpart) * 4 + nn) * 16 + g * 4 + rr;
-        if (col < Dv) orow[col] = acc[lb * 4 + nn][rr] * mul;
-      }
+      for (int rr = 0; rr < 4; ++rr) v[rr] = acc[lb * 4 + nn][rr] * mul;
+      if (half_out) Quad<unsigned short>::st(oh + col, v);
+      else Quad<float>::st(of + col, v);
+    }
   if (n_part > 1 && g == 0 && cpart == 0) {
     ws_ml[base * 2] = m; ws_ml[base * 2 + 1] = l;
   }
 }
 
 // out[row] = sum_p acc[row][p] e^(m_p - M) / sum_p l_p e^(m_p - M)
+template <typename TO>
 __global__ void __launch_bounds__(256) capped_attn_merge_kernel(
-    float* __restrict__ out, const float* __restrict__ ws_acc,
+    TO* __restrict__ out, long out_stride, const float* __restrict__ ws_acc,
     const float* __restrict__ ws_ml, int r, int n_part, int heads,
     const float* __restrict__ sink) {
   __shared__ float wgt[64];
@@ -391,7 +400,7 @@ __global__ void __launch_bounds__(256) capped_attn_merge_kernel(
     float a = 0.f;
 #pragma unroll 8
     for (int p = 0; p < n_part; ++p) a += base[(long)p * r + c] * wgt[p];
-    out[row * r + c] = a;
+    IO<TO>::st(out + (row / heads) * out_stride + (row % heads) * r + c, a);
   }
 }
 
@@ -405,7 +414,10 @@ int capped_attn_mfma_class(int D, int Dv) {
   return 0;
 }
 
-void launch_capped_attn_mfma(float* out, float* ws_acc, float* ws_ml,
+// out [tokens, heads*Dv], row stride out_stride, fp32 or bf16; rows 16 B / 8 B
+// aligned
+void launch_capped_attn_mfma(void* out, long out_stride, int out_bf16,
+                             float* ws_acc, float* ws_ml,
                              const unsigned short* q,
                              const unsigned short* k_cache,
                              const unsigned short* v_cache,
@@ -431,7 +443,8 @@ void launch_capped_attn_mfma(float* out, float* ws_acc, float* ws_ml,
   dim3 grid(blocks, n_part, n_kv);
 #define CM_LAUNCH(KQ, NO, CS)                                                \
   hipLaunchKernelGGL((capped_attn_mfma_kernel<KQ, NO, CS>), grid, dim3(256), \
-                     (size_t)(KQ * 2 + NO) * 1024, st, out, ws_acc, ws_ml,   \
+                     (size_t)(KQ * 2 + NO) * 1024, st, out, out_stride,      \
+                     out_bf16, ws_acc, ws_ml,                                \
                      q, k_cache, v_cache, block_tables, cu_q, seq_lens,      \
                      n_seqs, heads, n_kv, D, Dv, block_size, table_width,    \
                      scale, cap, q_stride, n_part, window, sink, keep_first, \
@@ -448,10 +461,16 @@ void launch_capped_attn_mfma(float* out, float* ws_acc, float* ws_ml,
   else CM_BY_CS(8, 16);
 #undef CM_BY_CS
 #undef CM_LAUNCH
-  if (n_part > 1)
-    hipLaunchKernelGGL(capped_attn_merge_kernel,
-                       dim3((unsigned)tokens * heads), dim3(256), 0, st, out,
-                       ws_acc, ws_ml, Dv, n_part, heads, sink);
+  if (n_part > 1 && out_bf16)
+    hipLaunchKernelGGL((capped_attn_merge_kernel<unsigned short>),
+                       dim3((unsigned)tokens * heads), dim3(256), 0, st,
+                       (unsigned short*)out, out_stride, ws_acc, ws_ml, Dv,
+                       n_part, heads, sink);
+  else if (n_part > 1)
+    hipLaunchKernelGGL((capped_attn_merge_kernel<float>),
+                       dim3((unsigned)tokens * heads), dim3(256), 0, st,
+                       (float*)out, out_stride, ws_acc, ws_ml, Dv, n_part,
+                       heads, sink);
 }
 
 }  // namespace hyb

@@ -9,7 +9,7 @@ namespace hyb {
 // One wavefront per token; z [T, E] are the fp32 router logits (an fp32 GEMM
 // upstream). Scores: sigmoid(z), or with `softmax` the softmax of z over all
 // experts. The choice runs on score + corr (corr nullable); the weights are
-// the plain scores, divided by their sum + 1e-20 with `normalize`.
+// the plain scores, divided by their sum + 1e-20 with `normalize`, times scale.
 // Experts form n_groups equal neighbouring groups; a group's score is the
 // sum of its two largest choice scores (the largest one with `group_max`);
 // only the `keep` best groups are eligible. ids/weights [T, top]: the
@@ -20,7 +20,7 @@ __global__ void moe_route_kernel(int* __restrict__ ids,
                                  const float* __restrict__ z, int E, int top,
                                  int n_groups, int keep, int softmax,
                                  const float* __restrict__ corr, int group_max,
-                                 int normalize) {
+                                 int normalize, float scale) {
   extern __shared__ float smem[];
   float* sc = smem;                 // [E] scores
   float* el = sc + E;               // [E] eligible choice score or -inf
@@ -86,7 +86,7 @@ __global__ void moe_route_kernel(int* __restrict__ ids,
     if (bi == 0x7fffffff) bi = 0;   // fewer eligible experts than top
     if (lane == 0) {
       ids[(long)t * top + kk] = bi;
-      wts[(long)t * top + kk] = sc[bi];
+      wts[(long)t * top + kk] = normalize ? sc[bi] : sc[bi] * scale;
       el[bi] = -INFINITY;
     }
     __syncthreads();
@@ -96,7 +96,7 @@ __global__ void moe_route_kernel(int* __restrict__ ids,
     for (int kk = 0; kk < top; ++kk) sum += wts[(long)t * top + kk];
     sum += 1e-20f;
     for (int kk = 0; kk < top; ++kk)
-      wts[(long)t * top + kk] = wts[(long)t * top + kk] / sum;
+      wts[(long)t * top + kk] = wts[(long)t * top + kk] / sum * scale;
   }
 }
 
@@ -134,12 +134,12 @@ __global__ void moe_combine_kernel(float* __restrict__ out,
 void launch_moe_route(int* ids, float* wts, const float* z, int tokens, int E,
                       int top, int n_groups, int keep, int softmax,
                       const float* corr, int group_max, int normalize,
-                      hipStream_t st) {
+                      float scale, hipStream_t st) {
   if (tokens == 0) return;
   const size_t lds = (size_t)(2 * E + n_groups) * sizeof(float);
   hipLaunchKernelGGL(moe_route_kernel, dim3(tokens), dim3(64), lds, st, ids,
                      wts, z, E, top, n_groups, keep, softmax, corr, group_max,
-                     normalize);
+                     normalize, scale);
 }
 
 template <typename T>

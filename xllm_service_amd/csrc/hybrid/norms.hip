@@ -99,20 +99,20 @@ __global__ void norm_sigmoid_gate_kernel(T* __restrict__ out,
 //   else:       out = o / rms_g(o) * w * act(gate)
 // act = silu or sigmoid; rms over `groups` equal consecutive parts; w has
 // w_period entries and repeats (w_period = n: one weight per column;
-// w_period = n / groups: the same weights for every group).
+// w_period = n / groups: the same weights for every group); w null: no weight.
 template <typename T>
 __global__ void gated_group_norm_kernel(
     T* __restrict__ out, const float* __restrict__ o,
     const float* __restrict__ w, int w_period, const T* __restrict__ gate,
     long gate_stride, float eps, int n, int groups, int act_silu,
-    int gate_first) {
+    int gate_first, long out_stride) {
   const int row = blockIdx.x;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int nw = blockDim.x >> 6;
   const int gs = n / groups;
   const float* orow = o + (long)row * n;
   const T* gr = gate + (long)row * gate_stride;
-  T* dst = out + (long)row * n;
+  T* dst = out + (long)row * out_stride;
   for (int g = wid; g < groups; g += nw) {
     float ss = 0.f;
     for (int i = lane; i < gs; i += 64) {
@@ -130,7 +130,8 @@ __global__ void gated_group_norm_kernel(
       const int c = g * gs + i;
       const float gv = IO<T>::ld(gr + c);
       const float a = act_silu ? siluf_(gv) : sigmoidf_(gv);
-      IO<T>::st(dst + c, orow[c] * a * rs * w[c % w_period]);
+      const float wc = w != nullptr ? w[c % w_period] : 1.0f;
+      IO<T>::st(dst + c, orow[c] * a * rs * wc);
     }
   }
 }
@@ -264,11 +265,12 @@ template <typename T>
 void launch_gated_group_norm(T* out, const float* o, const float* w,
                              int w_period, const T* gate, long gate_stride,
                              float eps, int rows, int n, int groups,
-                             int act_silu, int gate_first, hipStream_t st) {
+                             int act_silu, int gate_first, long out_stride,
+                             hipStream_t st) {
   if (rows == 0) return;
   hipLaunchKernelGGL((gated_group_norm_kernel<T>), dim3(rows), dim3(256), 0,
                      st, out, o, w, w_period, gate, gate_stride, eps, n,
-                     groups, act_silu, gate_first);
+                     groups, act_silu, gate_first, out_stride);
 }
 template <typename T>
 void launch_silu_mul(T* out, const T* x, long rows, int F, hipStream_t st) {
@@ -309,7 +311,8 @@ void launch_rope_interleaved(T* x, const long* pos, const double* inv_freq,
                                         hipStream_t);                         \
   template void launch_gated_group_norm<T>(T*, const float*, const float*,    \
                                            int, const T*, long, float, int,   \
-                                           int, int, int, int, hipStream_t);  \
+                                           int, int, int, int, long,          \
+                                           hipStream_t);                      \
   template void launch_rope_interleaved<T>(T*, const long*, const double*,    \
                                            float, int, int, int, long, long,  \
                                            int, int, hipStream_t);

@@ -5,12 +5,16 @@
 //   (u, v) -> (u cos a - v sin a, v cos a + u sin a),  a = pos * f_i,
 // with the pair (u, v) = entries (2i, 2i+1) of the head (`pairs`) or entries
 // (i, i + rot/2); then, with `unit`, the head is divided by its root mean
-// square sqrt(mean(x^2) + eps). cos and sin carry the factor mscale. Angle and sincos in fp64, the turn and the
-// norm in fp32. q' goes to a contiguous row tensor, k' and the untouched v
-// (when there is one) into the paged caches [blocks, n_kv, block, D | Dv] at
-// the token's slot (slot < 0: not stored). One workgroup per token; cos/sin
-// of the token are made once in LDS; a wave owns a head at a time and keeps
-// the head's entries in registers between the sum of squares and the store.
+// square sqrt(mean(x^2) + eps). With weights wq / wk (fp32 [D], the same for
+// every head) the norm comes BEFORE the turn: x / rms(x) * w. cos and sin carry
+// the factor mscale. Angle and sincos in fp64 (or read from a table [tokens,
+// rot] of cos | sin made once per step), the turn and the norm in fp32. q'
+// goes to a contiguous row tensor, k' and the untouched v (when there are
+// such) into the paged caches [blocks, n_kv, block, D | Dv] at the token's slot
+// (slot < 0: not stored); without k only the queries are prepared. One
+// workgroup per token; cos/sin of the token are made once in LDS; a wave owns
+// a head at a time and keeps the head's entries in registers between the sum
+// of squares and the store.
 //
 // polynorm: out = c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3 per row, N(u) = u /
 // sqrt(mean(u^2) + eps); powers element by element; fp32 inside.
@@ -30,22 +34,29 @@ __global__ void __launch_bounds__(256) rope_headnorm_store_kernel(
     const long* __restrict__ pos, const double* __restrict__ inv_freq, int rot,
     int pairs, int unit, float eps, int heads, int n_kv, int D, int Dv,
     T* __restrict__ k_cache, T* __restrict__ v_cache,
-    const long* __restrict__ slot_mapping, int block_size, float mscale) {
+    const long* __restrict__ slot_mapping, int block_size, float mscale,
+    const float* __restrict__ wq, const float* __restrict__ wk,
+    const float* __restrict__ table) {
   extern __shared__ float cs[];           // [rot/2] cos, [rot/2] sin
   const int t = blockIdx.x, tid = threadIdx.x;
   const int lane = tid & 63, wv = tid >> 6;
   const int half = rot >> 1;
-  for (int i = tid; i < half; i += 256) {
-    double s, c;
-    sincos((double)pos[t] * inv_freq[i], &s, &c);
-    cs[i] = (float)(c * mscale);
-    cs[half + i] = (float)(s * mscale);
+  if (table != nullptr) {
+    for (int i = tid; i < rot; i += 256) cs[i] = table[(long)t * rot + i];
+  } else {
+    for (int i = tid; i < half; i += 256) {
+      double s, c;
+      sincos((double)pos[t] * inv_freq[i], &s, &c);
+      cs[i] = (float)(c * mscale);
+      cs[half + i] = (float)(s * mscale);
+    }
   }
   __syncthreads();
   const long slot = slot_mapping[t];
   const long blk = slot >= 0 ? slot / block_size : 0;
   const long off = slot >= 0 ? slot % block_size : 0;
-  for (int u = wv; u < heads + n_kv; u += 4) {       // uniform per wave
+  const int units = k != nullptr ? heads + n_kv : heads;
+  for (int u = wv; u < units; u += 4) {              // uniform per wave
     const bool is_q = u < heads;
     const int g = u - heads;
     if (!is_q && slot < 0) continue;
@@ -53,20 +64,33 @@ __global__ void __launch_bounds__(256) rope_headnorm_store_kernel(
                         : k + (long)t * k_stride + (long)g * D;
     T* dst = is_q ? q_out + ((long)t * heads + u) * D
                   : k_cache + ((blk * n_kv + g) * block_size + off) * (long)D;
+    const float* hw = is_q ? wq : wk;                // norm before the turn
     float val[RH_MAX];
-    float ss = 0.f;
+    float ss = 0.f, pre = 1.f;
+    if (hw != nullptr) {
+#pragma unroll
+      for (int j = 0; j < RH_MAX; ++j) {
+        const int d = lane + 64 * j;
+        const float x = d < D ? IO<T>::ld(src + d) : 0.f;
+        ss += x * x;
+      }
+      pre = 1.0f / sqrtf(wave_reduce_sum(ss) / (float)D + eps);
+      ss = 0.f;
+    }
 #pragma unroll
     for (int j = 0; j < RH_MAX; ++j) {
       const int d = lane + 64 * j;
       float x = 0.f;
       if (d < D) {
         x = IO<T>::ld(src + d);
+        if (hw != nullptr) x = x * pre * hw[d];
         if (d < rot) {
           bool first; int i, pd;
           if (pairs) { first = !(d & 1); i = d >> 1; pd = d ^ 1; }
           else { first = d < half; i = first ? d : d - half;
                  pd = first ? d + half : d - half; }
-          const float y = IO<T>::ld(src + pd);
+          float y = IO<T>::ld(src + pd);
+          if (hw != nullptr) y = y * pre * hw[pd];
           const float c = cs[i], s = cs[half + i];
           x = first ? x * c - y * s : x * c + y * s;
         }
@@ -148,13 +172,15 @@ void launch_rope_headnorm_store(T* q_out, const T* q, const T* k, const T* v,
                                 int tokens, int heads, int n_kv, int D, int Dv,
                                 T* k_cache, T* v_cache,
                                 const long* slot_mapping, int block_size,
-                                float mscale, hipStream_t st) {
+                                float mscale, const float* wq,
+                                const float* wk, const float* table,
+                                hipStream_t st) {
   if (tokens == 0) return;
   hipLaunchKernelGGL((rope_headnorm_store_kernel<T>), dim3(tokens), dim3(256),
                      (size_t)(rot > 0 ? rot : 1) * sizeof(float), st, q_out, q,
                      k, v, q_stride, k_stride, v_stride, pos, inv_freq, rot,
                      pairs, unit, eps, heads, n_kv, D, Dv, k_cache, v_cache,
-                     slot_mapping, block_size, mscale);
+                     slot_mapping, block_size, mscale, wq, wk, table);
 }
 
 template <typename T>
@@ -179,7 +205,8 @@ void launch_gelu_tanh_gate(T* out, const T* g, const T* u, long rows, int F,
   template void launch_rope_headnorm_store<T>(                                \
       T*, const T*, const T*, const T*, long, long, long, const long*,        \
       const double*, int, int, int, float, int, int, int, int, int, T*, T*,   \
-      const long*, int, float, hipStream_t);                                  \
+      const long*, int, float, const float*, const float*, const float*,      \
+      hipStream_t);                                                           \
   template void launch_polynorm<T>(T*, const T*, const float*, float, long,   \
                                    int, long, hipStream_t);                   \
   template void launch_gelu_tanh_gate<T>(T*, const T*, const T*, long, int,   \

@@ -10,7 +10,7 @@ from typing import List, Optional
 @dataclass
 class ModelConfig:
     name: str = "llama"
-    architecture: str = "llama"   # llama | opt | qwen2 | qwen2_vl | pugovik | dunusun | tosipel | gararax | nikedra
+    architecture: str = "llama"   # llama | opt | qwen2 | qwen2_vl | pugovik | dunusun | tosipel | gararax | nikedra | zokanex
     vocab_size: int = 128256
     hidden_size: int = 4096
     intermediate_size: int = 14336
@@ -383,6 +383,51 @@ def nikedra_from_dict(d: dict, name: str = "nikedra",
         max_position=1 << 20, layers=layers, model_dir=model_dir)
 
 
+@dataclass
+class ZokanexConfig(ModelConfig):
+    """Zokanex: layers of windowed grouped-head softmax attention with a
+    weighted norm of every query and key head (`attention`; a layer may read
+    an earlier layer's keys and values) or of retention, a linear attention
+    with a fixed decay per head (`retention`); mixer and feed-forward read the
+    same normed residual and are added to it together; dense GELU-gated or
+    routed-expert feed-forwards with a gated shared expert."""
+    layers: List[HybridLayerConfig] = field(default_factory=list)
+    embed_scale: float = 1.0
+    model_dir: Optional[str] = None     # weights live here (None = random)
+
+    @property
+    def has_recurrent_state(self) -> bool:
+        return any(l.type == "retention" for l in self.layers)
+
+
+def zokanex_from_dict(d: dict, name: str = "zokanex",
+                      model_dir: Optional[str] = None) -> ZokanexConfig:
+    layers = [HybridLayerConfig(type=l["type"], mixer=dict(l["mixer"]),
+                                mlp=l.get("mlp"))
+              for l in d["layers"]]
+    for i, l in enumerate(layers):
+        if l.type not in ("attention", "retention"):
+            raise ValueError(f"layer {i}: unknown mixer type {l.type!r}")
+        if l.mlp is not None and l.mlp.get("kind") not in ("dense", "moe"):
+            raise ValueError(f"layer {i}: unknown feed-forward kind")
+        src = l.mixer.get("kv_from")
+        if src is not None:
+            s = layers[src] if 0 <= src < i else None
+            if (s is None or s.type != "attention" or l.type != "attention"
+                    or s.mixer.get("kv_from") is not None
+                    or any(s.mixer[n] != l.mixer[n]
+                           for n in ("kv_heads", "dim", "vdim"))):
+                raise ValueError(f"layer {i}: kv_from {src} is not an earlier "
+                                 "attention layer with its own keys of the "
+                                 "same sizes")
+    return ZokanexConfig(
+        name=name, architecture="zokanex", vocab_size=int(d["vocab"]),
+        hidden_size=int(d["width"]), num_layers=len(layers),
+        rms_eps=float(d["norm"]["eps"]),
+        embed_scale=float((d.get("embedding") or {}).get("scale", 1.0)),
+        max_position=1 << 20, layers=layers, model_dir=model_dir)
+
+
 def load_model_dir(path: str) -> ModelConfig:
     """Read <path>/config.json and pick the config class by its
     `architecture` field."""
@@ -404,6 +449,9 @@ def load_model_dir(path: str) -> ModelConfig:
     if arch == "nikedra":
         return nikedra_from_dict(d, name=os.path.basename(
             os.path.normpath(path)) or "nikedra", model_dir=path)
+    if arch == "zokanex":
+        return zokanex_from_dict(d, name=os.path.basename(
+            os.path.normpath(path)) or "zokanex", model_dir=path)
     raise ValueError(f"{path}: unsupported architecture "
                      f"{d.get('architecture')!r}")
 
@@ -651,6 +699,53 @@ PRESETS.update({
     # bench stacks at the width of real deployments (random weights)
     "nikedra-2k": _nikedra_preset("nikedra-2k", 2048, 8),
     "nikedra-4k": _nikedra_preset("nikedra-4k", 4096, 8),
+})
+
+
+def _zokanex_preset(name, width, n_layers, vocab=32000, head=128, window=1024,
+                    experts=16, top=2):
+    """Synthetic Zokanex stacks for benchmarks: per group of four layers a
+    windowed attention layer, two retention layers and an attention layer that
+    reads the first one's keys through a window of half the size; dense and
+    routed feed-forwards in turn."""
+    heads = max(width // head, 1)
+    dense = dict(kind="dense", ff=3 * width // 2)
+    groups = 4 if experts % 4 == 0 and experts >= 8 else 2
+    moe = dict(kind="moe", expert=dict(ff=width // 2),
+               router=dict(experts=experts, top=top, scale=1.25,
+                           groups=dict(count=groups, keep=groups // 2)),
+               shared=dict(ff=width // 2))
+    layers, own = [], None
+    for i in range(n_layers):
+        k, mlp = i % 4, moe if i % 2 else dense
+        if k in (0, 3):
+            mixer = dict(heads=heads, kv_heads=max(heads // 4, 1), dim=head,
+                         vdim=head, scale=head ** -0.5,
+                         mask=dict(size=window if k == 0 else window // 2),
+                         rot=dict(base=10000.0, dims=head))
+            if k == 3:
+                mixer["kv_from"] = own
+            else:
+                own = i
+            layers.append(dict(type="attention", mixer=mixer, mlp=mlp))
+        else:
+            decay = [1.0 - 2.0 ** -(4 + 6 * h / max(heads - 1, 1))
+                     for h in range(heads)]
+            layers.append(dict(type="retention", mlp=mlp, mixer=dict(
+                heads=heads, dim=head, vdim=head, decay=decay,
+                rot=dict(base=10000.0, dims=head))))
+    return zokanex_from_dict(dict(
+        architecture="Zokanex", vocab=vocab, width=width, layers=layers,
+        norm=dict(eps=1e-6), embedding=dict(scale=2.0)), name=name)
+
+
+PRESETS.update({
+    # CPU-test sized stack
+    "zokanex-tiny": _zokanex_preset("zokanex-tiny", 64, 4, vocab=256, head=16,
+                                    window=20, experts=6),
+    # bench stacks at the width of real deployments (random weights)
+    "zokanex-2k": _zokanex_preset("zokanex-2k", 2048, 8),
+    "zokanex-4k": _zokanex_preset("zokanex-4k", 4096, 8),
 })
 
 

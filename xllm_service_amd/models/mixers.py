@@ -38,12 +38,19 @@ GroupedAttention       softmax attention with grouped key/value heads whose
                        turn, a sliding window that also keeps the first
                        tokens, chunks instead of a window, a sink of score 0,
                        one score multiplier per head, keys read as values,
-                       sigmoid gate per element or per head.
+                       sigmoid gate per element or per head, weighted RMS norm
+                       of q and k per head before the turn, keys and values
+                       of an earlier layer.
+Retention              S <- decay * S + k v^T, o = S^T q with one fixed decay
+                       per head and rotary positions on q and k; every
+                       head's o divided by its root mean square, SiLU gate.
 InputConvolution       h + causal convolution of h over time, in front of a
                        mixer's projections.
 
 All take the slice of a merged input projection that belongs to them and
-return the mixer output in the model dtype. Sizes and constants are
+return the mixer output in the model dtype. With project=False (where offered)
+the output projection is the caller's: `heads_out(.., out)` writes the heads'
+outputs, o_width columns, into rows the caller chose. Sizes and constants are
 constructor arguments.
 """
 from __future__ import annotations
@@ -267,6 +274,16 @@ def _halves(meta: AttnMetadata, aux):
                     meta.decode_state_slots, meta.decode_seq_lens,
                     meta.decode_block_tables, 1))
     return out
+
+
+def rotary_table(mixer, positions, aux):
+    """cos | sin of the step's positions at the mixer's frequencies, made by
+    the first layer of a step that needs them and shared with the others."""
+    tables = aux.setdefault("rotary", {})
+    key = (mixer.rot_key, mixer.mscale)
+    if key not in tables:
+        tables[key] = hops.rope_table(positions, mixer.inv_freq, mixer.mscale)
+    return tables[key]
 
 
 class InputConvolution(nn.Module):
@@ -610,8 +627,8 @@ class GatedDeltaRule(nn.Module):
 
 class GroupedAttention(nn.Module):
     """in_proj rows: [q: heads*dim | k: kv_heads*dim | v: kv_heads*vdim
-    (absent with values_are_keys) | g: heads*vdim (with gated), heads (with
-    head_gated)].
+    (absent with values_are_keys; k and v absent with kv_from) | g: heads*vdim
+    (with gated), heads (with head_gated)].
 
     rot: {base, dims, scaling?} or None; rot_pairs: entries (2i, 2i+1) turn
     together, else (i, i + dims/2). unit_norm: q and k are divided by their
@@ -623,7 +640,10 @@ class GroupedAttention(nn.Module):
     one such number per head. chunked: `window` is the size of the chunks,
     counted from position 0, that keep to themselves. yarn: rot's `scaling`
     is that of scaled_rope_frequencies (ramp over the pair index, cos/sin
-    multiplier), else that of banded_rope_frequencies."""
+    multiplier), else that of banded_rope_frequencies. head_norm: q and k are
+    divided by their root mean square per head and multiplied by one weight
+    vector each, shared by the heads, before the turn. kv_from: the layer whose
+    cached keys and values are read instead of own ones."""
 
     def __init__(self, width: int, heads: int, kv_heads: int, dim: int,
                  vdim: int, rot: Optional[dict], rot_pairs: bool,
@@ -631,7 +651,9 @@ class GroupedAttention(nn.Module):
                  dtype, *, unit_norm: bool = False, zero_sink: bool = False,
                  head_scale: bool = False, values_are_keys: bool = False,
                  gated: bool = False, head_gated: bool = False,
-                 chunked: bool = False, yarn: bool = False):
+                 chunked: bool = False, yarn: bool = False,
+                 head_norm: bool = False, kv_from: Optional[int] = None,
+                 project: bool = True):
         super().__init__()
         if heads % kv_heads:
             raise ValueError("heads must be a multiple of kv_heads")
@@ -657,8 +679,13 @@ class GroupedAttention(nn.Module):
         else:
             inv_freq = banded_rope_frequencies(rot)
         self.register_buffer("inv_freq", inv_freq, persistent=False)
-        self.cq, self.ck = heads * dim, kv_heads * dim
-        self.cv = 0 if values_are_keys else kv_heads * vdim
+        self.rot_key = tuple(inv_freq.tolist())
+        self.kv_from = kv_from
+        self.cq = heads * dim
+        self.ck = 0 if kv_from is not None else kv_heads * dim
+        self.cv = 0 if values_are_keys or kv_from is not None \
+            else kv_heads * vdim
+        self.o_width = heads * vdim
         self.gate_cols = vdim if head_gated else 1   # columns per gate entry
         self.g_width = heads * vdim // self.gate_cols if self.gated else 0
         self.in_width = self.cq + self.ck + self.cv + self.g_width
@@ -670,32 +697,50 @@ class GroupedAttention(nn.Module):
             self.sink = None
         self.head_scale = nn.Parameter(torch.ones(heads, **f32)) \
             if head_scale else None
-        self.o_proj = nn.Parameter(torch.empty(width, heads * vdim,
-                                               dtype=dtype))
+        self.q_norm = nn.Parameter(torch.ones(dim, **f32)) \
+            if head_norm else None
+        self.k_norm = nn.Parameter(torch.ones(dim, **f32)) \
+            if head_norm and kv_from is None else None
+        if project:
+            self.o_proj = nn.Parameter(torch.empty(width, self.o_width,
+                                                   dtype=dtype))
+        elif self.gated:
+            raise ValueError("the output gate needs the own projection")
 
     def cache_spec(self):
+        if self.kv_from is not None:
+            return SharedCache(self.kv_from)
         return PagedKV(self.kv_heads, self.dim, self.vdim,
                        values_are_keys=self.values_are_keys)
 
-    def forward(self, proj, positions, cache, meta: AttnMetadata, aux):
+    def heads_out(self, proj, positions, cache, meta: AttnMetadata, aux, out):
+        """The heads' outputs [T, o_width] into `out`: fp32, or rows of a wider
+        tensor in the model dtype."""
         k_cache, v_cache = cache
-        T, cq, ck, cv = proj.shape[0], self.cq, self.ck, self.cv
+        cq, ck, cv = self.cq, self.ck, self.cv
         H = self.heads
-        v_in = proj[:, cq + ck:cq + ck + cv] if cv else None
         q = hops.rope_headnorm_store(
-            proj[:, :cq], proj[:, cq:cq + ck], v_in, positions, self.inv_freq,
-            self.rot_dims, self.rot_pairs, self.unit_norm, self.eps, H,
-            self.kv_heads, k_cache, v_cache, meta.slot_mapping, self.mscale)
-        o = torch.empty(T, H, self.vdim, dtype=torch.float32,
-                        device=proj.device)
+            proj[:, :cq], proj[:, cq:cq + ck] if ck else None,
+            proj[:, cq + ck:cq + ck + cv] if cv else None, positions,
+            self.inv_freq, self.rot_dims, self.rot_pairs, self.unit_norm,
+            self.eps, H, self.kv_heads, k_cache, v_cache, meta.slot_mapping,
+            self.mscale, self.q_norm, self.k_norm,
+            rotary_table(self, positions, aux) if self.rot_dims else None)
         for rows, cu_q, _, _, seq_lens, tables, _ in _halves(meta, aux):
             hops.capped_attn(q[rows], k_cache, v_cache, tables, cu_q,
-                             seq_lens, H, self.scale, 0.0, o[rows],
+                             seq_lens, H, self.scale, 0.0, out[rows],
                              window=self.window, sink=self.sink,
                              keep_first=self.keep_first,
                              head_scale=self.head_scale,
                              chunked=self.chunked)
-        o = o.view(T, H * self.vdim)
+        return out
+
+    def forward(self, proj, positions, cache, meta: AttnMetadata, aux):
+        T, cq, ck, cv = proj.shape[0], self.cq, self.ck, self.cv
+        o = torch.empty(T, self.heads, self.vdim, dtype=torch.float32,
+                        device=proj.device)
+        o = self.heads_out(proj, positions, cache, meta, aux, o) \
+            .view(T, self.o_width)
         if self.gated:
             y = hops.norm_sigmoid_gate(
                 o, None, proj[:, cq + ck + cv:self.in_width], 0.0, proj.dtype,
@@ -703,3 +748,53 @@ class GroupedAttention(nn.Module):
         else:
             y = o.to(proj.dtype)
         return F.linear(y, self.o_proj)
+
+
+class Retention(nn.Module):
+    """in_proj rows: [q: heads*dim | k: heads*dim | v: heads*vdim |
+    g: heads*vdim]. decay: one number per head. rot: {base, dims} (half layout)
+    or None; k is multiplied by dim^-1/2 after the turn."""
+
+    def __init__(self, width: int, heads: int, dim: int, vdim: int, decay,
+                 rot: Optional[dict], norm_eps: float, dtype, *,
+                 project: bool = True):
+        super().__init__()
+        if len(decay) != heads:
+            raise ValueError("one decay per head")
+        self.heads, self.dim, self.vdim, self.eps = heads, dim, vdim, norm_eps
+        self.register_buffer("decay", torch.tensor(decay, dtype=torch.float32),
+                             persistent=False)
+        rot_dims = int(rot["dims"]) if rot else 0
+        if rot_dims > dim or rot_dims % 2:
+            raise ValueError("rotary dims must be even and <= dim")
+        inv_freq = banded_rope_frequencies(rot) if rot_dims \
+            else torch.zeros(0, dtype=torch.float64)
+        self.mscale = 1.0
+        self.register_buffer("inv_freq", inv_freq, persistent=False)
+        self.rot_key = tuple(inv_freq.tolist())
+        self.qk_width, self.o_width = heads * dim, heads * vdim
+        self.in_width = 2 * self.qk_width + 2 * self.o_width
+        if project:
+            self.o_proj = nn.Parameter(torch.empty(width, self.o_width,
+                                                   dtype=dtype))
+
+    def cache_spec(self):
+        return RecurrentState(self.heads, self.dim, self.vdim)
+
+    def heads_out(self, proj, positions, state, meta: AttnMetadata, aux, out):
+        """Normed and gated head outputs [T, o_width] into rows of `out`."""
+        a, b = self.qk_width, self.o_width
+        table = rotary_table(self, positions, aux)
+        for rows, cu_q, ctx, slots, _, _, _ in _halves(meta, aux):
+            p = proj[rows]
+            hops.retention(p[:, :a], p[:, a:2 * a], p[:, 2 * a:2 * a + b],
+                           p[:, 2 * a + b:self.in_width], table[rows],
+                           self.dim ** -0.5, self.decay, state, slots, cu_q,
+                           ctx, self.eps, out[rows])
+        return out
+
+    def forward(self, proj, positions, state, meta: AttnMetadata, aux):
+        y = torch.empty(proj.shape[0], self.o_width, dtype=proj.dtype,
+                        device=proj.device)
+        return F.linear(self.heads_out(proj, positions, state, meta, aux, y),
+                        self.o_proj)

@@ -10,13 +10,15 @@ Options: softmax scores over all experts, a correction added to the scores
 for the choice only, groups scored by their best expert, weights divided by
 their sum, `identity` further router outputs that stand for experts without
 tensors whose output is their input, a shared expert of the same form that
-every token uses (added to the routed sum in fp32), experts without a gate
+every token uses (added to the routed sum in fp32), a multiplier of the
+weights, experts without a gate
 (down(gelu(up h)), exact GELU), and the router weight on an expert's input
 instead of its output (the up-projection is linear, so the activation kernel
 applies the weight to its rows).
 
 Expert matrices are kept [expert, in, out], the contiguous right operand of a
-batched product.
+batched product. `dispatch()` stops before the combine, for layers that add
+the weighted expert outputs to the residual themselves.
 
 Two execution shapes over the same weights, both ending in the fp32 combine
 kernel: few tokens (decode batches, graph capture) run every expert as one
@@ -41,7 +43,8 @@ class RoutedExperts(nn.Module):
                  *, identity: int = 0, softmax: bool = False,
                  correction: bool = False, group_max: bool = False,
                  normalize: bool = False, shared_ff: int = 0,
-                 gated: bool = True, weight_input: bool = False):
+                 gated: bool = True, weight_input: bool = False,
+                 scale: float = 1.0):
         super().__init__()
         n_all = experts + identity
         if n_all % n_groups or keep > n_groups or \
@@ -50,6 +53,7 @@ class RoutedExperts(nn.Module):
         self.width, self.ff, self.experts, self.top = width, ff, experts, top
         self.n_groups, self.keep = n_groups, keep
         self.identity, self.softmax = identity, softmax
+        self.scale = float(scale)
         self.group_max, self.normalize = group_max, normalize
         if weight_input and (gated or identity or shared_ff):
             raise ValueError("weights on the input: plain experts only")
@@ -88,16 +92,25 @@ class RoutedExperts(nn.Module):
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         """h [T, width] (model dtype) -> fp32 [T, width]."""
-        T, E = h.shape[0], self.experts
-        ids, wts = hops.moe_route(
-            h, self.router, self.top, self.n_groups, self.keep,
-            softmax=self.softmax, correction=self.correction,
-            group_max=self.group_max, normalize=self.normalize)
+        y, rows, mix = self.dispatch(h)
         extra = None
         if self.shared_ff:
             extra = F.linear(hops.silu_mul(F.linear(h, self.shared_gate_up)),
                              self.shared_down)
-        ident = h if self.identity else None
+        return hops.moe_combine(y, rows, mix, h.shape[0],
+                                h if self.identity else None, extra)
+
+    def dispatch(self, h: torch.Tensor):
+        """Route h and run the chosen experts. Returns (y [.., width], rows
+        int32 [T, top], weights fp32 [T, top] or None): the routed sum of
+        token t is sum_k weights[t, k] * y[rows[t, k]], a negative row standing
+        for an identity expert; weights None: they are in y already."""
+        T, E = h.shape[0], self.experts
+        ids, wts = hops.moe_route(
+            h, self.router, self.top, self.n_groups, self.keep,
+            softmax=self.softmax, correction=self.correction,
+            group_max=self.group_max, normalize=self.normalize,
+            scale=self.scale)
         win = self.weight_input
         mix = None if win else wts         # what the combine multiplies by
         capturing = h.is_cuda and torch.cuda.is_current_stream_capturing()
@@ -110,7 +123,7 @@ class RoutedExperts(nn.Module):
                                           device=h.device)[:, None]
             if self.identity:
                 rows = torch.where(ids >= E, -1, rows)
-            return hops.moe_combine(y, rows, mix, T, ident, extra)
+            return y, rows, mix
         # identity choices sort behind every expert and take no rows
         flat = ids.reshape(-1).long()
         order = torch.argsort(flat, stable=True)
@@ -123,9 +136,7 @@ class RoutedExperts(nn.Module):
         rows = torch.full((T * self.top,), -1, dtype=torch.int32,
                           device=h.device)
         if total == 0:
-            y = h.new_zeros(1, self.width)
-            return hops.moe_combine(y, rows.view(T, self.top), mix, T, ident,
-                                    extra)
+            return h.new_zeros(1, self.width), rows.view(T, self.top), mix
         scale = wts.reshape(-1)[order] if win else None      # per sorted row
         if cap * E <= 1.5 * total + 16 * E:
             # near-even load: pad every expert to `cap` rows and run all of
@@ -141,9 +152,7 @@ class RoutedExperts(nn.Module):
             z = torch.bmm(xs.view(E, cap, self.width), self.w_in)
             y = torch.bmm(self._act(z, scale), self.w_down)
             rows[order] = dest.to(torch.int32)
-            return hops.moe_combine(y.view(-1, self.width),
-                                    rows.view(T, self.top), mix, T, ident,
-                                    extra)
+            return y.view(-1, self.width), rows.view(T, self.top), mix
         xs = h[order // self.top]
         ys = torch.empty(total, self.width, dtype=h.dtype, device=h.device)
         at = 0
@@ -155,5 +164,4 @@ class RoutedExperts(nn.Module):
                 ys[seg] = act @ self.w_down[e]
                 at += n
         rows[order] = torch.arange(total, dtype=torch.int32, device=h.device)
-        return hops.moe_combine(ys, rows.view(T, self.top), mix, T, ident,
-                                extra)
+        return ys, rows.view(T, self.top), mix

@@ -33,12 +33,15 @@ def create_model(cfg: ModelConfig, dtype=torch.bfloat16):
     if cfg.architecture == "nikedra":
         from .nikedra import NikedraForCausalLM
         return NikedraForCausalLM(cfg, dtype=dtype)
+    if cfg.architecture == "zokanex":
+        from .zokanex import ZokanexForCausalLM
+        return ZokanexForCausalLM(cfg, dtype=dtype)
     raise ValueError(f"unknown architecture {cfg.architecture}")
 
 
 def required_extensions(cfg: ModelConfig):
     """In-tree HIP extension modules the model's GPU path loads."""
     if cfg.architecture in ("pugovik", "dunusun", "tosipel", "gararax",
-                            "nikedra"):
+                            "nikedra", "zokanex"):
         return ["_ops_hybrid"]
     return ["_ops"]

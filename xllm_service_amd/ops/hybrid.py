@@ -2,7 +2,9 @@
 recurrent state, grouped RMS norms, gated residuals, routed experts;
 residual streams, short convolutions, gated recurrences, soft-capped and
 windowed paged attention; post-norm residual, whole-row q/k norm with
-rotate-half positions, the gated delta rule; depth average of the residual.
+rotate-half positions, the gated delta rule; depth average of the residual;
+retention, and the joint residual update of layers whose mixer and feed-forward
+read one norm.
 
 Same policy as the rest of `ops`: on a GPU the HIP extension (`_ops_hybrid`)
 is the only path and its absence raises; on CPU the fp32 torch references in
@@ -137,23 +139,24 @@ def decay_attn(q, k, v, decay, state, slots, cu_q, ctx_lens, out,
 
 def moe_route(h, w_router, top: int, n_groups: int, keep: int, *,
               softmax: bool = False, correction=None, group_max: bool = False,
-              normalize: bool = False):
+              normalize: bool = False, scale: float = 1.0):
     """Router: fp32 logits h @ w_router^T (a true-fp32 library GEMM on the
     GPU; h enters as stored, i.e. possibly bf16-rounded), then the scores
     (sigmoid, or softmax over all experts) and the group-limited top-k
     selection kernel. correction fp32 [experts] is added to the scores for
     the choice only; group_max scores a group by its best expert instead of
-    its two best; normalize divides the chosen weights by their sum."""
+    its two best; normalize divides the chosen weights by their sum; scale
+    multiplies them."""
     if h.is_cuda:
         T = h.shape[0]
         z = torch.matmul(h.float(), w_router.t())
         ids = torch.empty(T, top, dtype=torch.int32, device=h.device)
         wts = torch.empty(T, top, dtype=torch.float32, device=h.device)
         _hyb().moe_route(ids, wts, z, top, n_groups, keep, softmax,
-                         correction, group_max, normalize)
+                         correction, group_max, normalize, scale)
         return ids, wts
     return ref.moe_route(h, w_router, top, n_groups, keep, softmax,
-                         correction, group_max, normalize)
+                         correction, group_max, normalize, scale)
 
 
 def moe_combine(y, rows, wts, tokens: int, ident=None, extra=None):
@@ -292,6 +295,7 @@ def gated_recurrence(kind: int, q, k, v, g, p0, p1, p2, c0: float, c1: float,
 
 def gated_group_norm(o, w, gate, eps: float, groups: int, *, act_silu: bool,
                      gate_first: bool, out_dtype):
+    """w None: no weight."""
     if o.is_cuda:
         out = torch.empty(o.shape, dtype=out_dtype, device=o.device)
         _hyb().gated_group_norm(out, o, w, gate, eps, groups, act_silu,
@@ -306,7 +310,8 @@ def capped_attn(q, k_cache, v_cache, block_tables, cu_q, seq_lens,
                 sink: Optional[torch.Tensor] = None, keep_first: int = 0,
                 head_scale: Optional[torch.Tensor] = None,
                 chunked: bool = False):
-    """out fp32 [T, heads, Dv] (written). cu_q None: decode rows. window > 0
+    """out (written): fp32 [T, heads, Dv], or [T, heads*Dv] rows of a wider
+    tensor in q's dtype. cu_q None: decode rows. window > 0
     limits a query to the last `window` keys (itself included) and, with
     keep_first, the first keep_first keys of the sequence; chunked: `window`
     is the size of the chunks, counted from position 0, that the sequence
@@ -322,7 +327,7 @@ def capped_attn(q, k_cache, v_cache, block_tables, cu_q, seq_lens,
         return out
     out.copy_(ref.capped_attn(q, k_cache, v_cache, block_tables, cu_q,
                               seq_lens, heads, scale, cap, window, sink,
-                              keep_first, head_scale, chunked))
+                              keep_first, head_scale, chunked).view(out.shape))
     return out
 
 
@@ -386,22 +391,26 @@ def gelu_tanh_mul(x):
 def rope_headnorm_store(q, k, v, positions, inv_freq, rot_dims: int,
                         pairs: bool, unit_norm: bool, eps: float, heads: int,
                         kv_heads: int, k_cache, v_cache, slot_mapping,
-                        mscale: float = 1.0):
+                        mscale: float = 1.0, q_w=None, k_w=None, table=None):
     """Rotary turn on the first rot_dims entries of every head of q [T,
     heads*D] and k [T, kv_heads*D] (`pairs`: entries 2i / 2i+1, else i / i +
-    rot_dims/2; cos/sin scaled by mscale), then with unit_norm each head divided by its root mean
-    square. Returns the new q as a contiguous tensor; k and v (None: the
-    values are the keys) go into the paged caches at the tokens' slots."""
+    rot_dims/2; cos/sin scaled by mscale), then with unit_norm each head
+    divided by its root mean square. q_w, k_w (fp32 [D]): each head is
+    divided by its root mean square and multiplied by them BEFORE the turn.
+    Returns the new q as a contiguous tensor; k and v (v None: the values are
+    the keys; both None: queries only) go into the paged caches at the
+    tokens' slots. table: rope_table() of the rows, if there is one."""
     if q.is_cuda:
         out = torch.empty(q.shape, dtype=q.dtype, device=q.device)
         _hyb().rope_headnorm_store(out, q, k, v, positions, inv_freq,
                                    rot_dims, pairs, unit_norm, eps, heads,
                                    kv_heads, k_cache, v_cache, slot_mapping,
-                                   mscale)
+                                   mscale, q_w, k_w, table)
         return out
     return ref.rope_headnorm_store(q, k, v, positions, inv_freq, rot_dims,
                                    pairs, unit_norm, eps, heads, kv_heads,
-                                   k_cache, v_cache, slot_mapping, mscale)
+                                   k_cache, v_cache, slot_mapping, mscale,
+                                   q_w, k_w)
 
 
 def polynorm(z, coef, eps: float):
@@ -462,3 +471,70 @@ def gelu_scaled(x, scale=None, ids=None, wts=None):
         _hyb().gelu_scaled(out, x, scale, ids, wts)
         return out
     return ref.gelu_scaled(x, scale, ids, wts)
+
+
+# ---- retention, joint residual update ----------------------------------------
+def rope_table(positions, inv_freq, mscale: float = 1.0):
+    """fp32 [T, 2 * len(inv_freq)]: cos | sin of position * frequency (fp64
+    angles), times mscale; made once per step for every layer that turns by
+    these frequencies."""
+    if positions.is_cuda:
+        t = torch.empty(positions.numel(), 2 * inv_freq.numel(),
+                        dtype=torch.float32, device=positions.device)
+        _hyb().rope_table(t, positions, inv_freq, mscale)
+        return t
+    return ref.rope_table_rows(positions, inv_freq, mscale)
+
+
+def retention(q, k, v, gate, table, k_scale: float, decay, state, slots, cu_q,
+              ctx_lens, eps: float, out):
+    """out [T, H*Dv] (written, rows of a wider tensor are fine): the gated
+    head norm of S^T q with S <- decay_h S + k v^T; see ref.retention. q, k,
+    v, gate are row views of the projections, turned by `table` inside; state
+    fp32 [slots, H, D, Dv] in place. cu_q None: decode rows."""
+    if q.is_cuda:
+        _hyb().retention(out, q, k, v, gate, table, k_scale, decay, state,
+                         slots, cu_q, ctx_lens, eps)
+        return out
+    out.copy_(ref.retention(q, k, v, gate, table, k_scale, decay, state,
+                            slots, cu_q, ctx_lens, eps))
+    return out
+
+
+def glu_rows(g, u, out, *, gelu: bool, row_gate=None):
+    """out = act(g) * u, times sigmoid(row_gate) [T, 1] if given; act = tanh
+    GELU or SiLU; g, u, out [T, F] row views of one dtype."""
+    if g.is_cuda:
+        _hyb().glu_rows(out, g, u, row_gate, gelu)
+        return out
+    return out.copy_(ref.glu_rows(g, u, gelu, row_gate))
+
+
+def embed_norm(table, ids, scale: float, w, eps: float, out_dtype):
+    """x = scale * table[ids] in fp32 (ids None: scale * table, one row per
+    token) and its norm x / rms(x) * w in out_dtype, from one pass."""
+    if table.is_cuda:
+        T = table.shape[0] if ids is None else ids.numel()
+        x = torch.empty(T, table.shape[1], dtype=torch.float32,
+                        device=table.device)
+        h = torch.empty(x.shape, dtype=out_dtype, device=table.device)
+        _hyb().join_norm(x, h, True, table, ids, scale, None, None, None, w,
+                         eps)
+        return x, h
+    x = (table if ids is None else table[ids]).float() * scale
+    return x, ref.rmsnorm(x, w, eps).to(out_dtype)
+
+
+def join_norm_(x, y, experts, w, eps: float):
+    """x (fp32 [T, W], in place) += y + the routed experts' weighted outputs
+    (experts: (e [.., W], rows int32 [T, top], wts fp32) or None, a negative
+    row adds nothing); returns x / rms(x) * w in y's dtype."""
+    e, rows, wts = experts if experts is not None else (None, None, None)
+    if x.is_cuda:
+        h = torch.empty(x.shape, dtype=y.dtype, device=x.device)
+        _hyb().join_norm(x, h, False, y, None, 1.0, e, rows, wts, w, eps)
+        return h
+    x.add_(y.float())
+    if e is not None:
+        x.add_(moe_combine(e, rows, wts * (rows >= 0), x.shape[0]))
+    return ref.rmsnorm(x, w, eps).to(y.dtype)

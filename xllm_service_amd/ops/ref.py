@@ -294,11 +294,12 @@ def decay_linear_attn(q, k, v, decay, state, slots, cu_q, ctx_lens):
 
 
 def moe_route(h, w_router, top, n_groups, keep, softmax=False,
-              correction=None, group_max=False, normalize=False):
+              correction=None, group_max=False, normalize=False, scale=1.0):
     """Top-k routing with group limiting. Scores: sigmoid of the fp32 logits,
     or their softmax over all experts. The choice is made on the scores plus
     `correction` (when given); the weights are the plain scores of the
-    chosen, divided by their sum (+ 1e-20) with `normalize`. Experts form
+    chosen, divided by their sum (+ 1e-20) with `normalize`, times scale.
+    Experts form
     n_groups equal neighbouring groups, scored by the sum of their two
     largest choice scores (by the largest one with `group_max`); only the
     best `keep` groups are eligible. Returns (ids [T, top] int32, weights
@@ -320,7 +321,7 @@ def moe_route(h, w_router, top, n_groups, keep, softmax=False,
     wts = s.gather(1, idx)
     if normalize:
         wts = wts / (wts.sum(-1, keepdim=True) + 1e-20)
-    return idx.to(torch.int32), wts
+    return idx.to(torch.int32), wts * scale
 
 
 def silu_mul(x):
@@ -451,7 +452,7 @@ def gated_recurrence(kind, q, k, v, g, p0, p1, p2, c0, c1, state, slots, cu_q,
 def gated_group_norm(o, w, gate, eps, groups, act_silu, gate_first,
                      out_dtype):
     """RMS norm over `groups` equal parts of fp32 o [rows, n], times w (n
-    or n/groups entries, repeating), with gate silu/sigmoid applied before
+    or n/groups entries, repeating; None: 1), with gate silu/sigmoid applied before
     or after the norm."""
     act = torch.nn.functional.silu if act_silu else torch.sigmoid
     a = act(gate.float())
@@ -459,10 +460,10 @@ def gated_group_norm(o, w, gate, eps, groups, act_silu, gate_first,
     rows, n = z.shape
     zg = z.view(rows, groups, n // groups)
     zg = zg * torch.rsqrt(zg.pow(2).mean(-1, keepdim=True) + eps)
-    wf = w.float()
-    if wf.numel() != n:
-        wf = wf.repeat(groups)
-    z = zg.reshape(rows, n) * wf
+    z = zg.reshape(rows, n)
+    if w is not None:
+        wf = w.float()
+        z = z * (wf if wf.numel() == n else wf.repeat(groups))
     if not gate_first:
         z = z * a
     return z.to(out_dtype)
@@ -633,16 +634,19 @@ def gelu_tanh_mul(x):
 # ---------------------------------------------------------------------------
 def rope_headnorm_store(q, k, v, positions, inv_freq, rot_dims, pairs,
                         unit_norm, eps, heads, kv_heads, k_cache, v_cache,
-                        slot_mapping, mscale=1.0):
+                        slot_mapping, mscale=1.0, q_w=None, k_w=None):
     """q [T, heads*D], k [T, kv_heads*D]: rotary turn on the first rot_dims
     entries of every head (`pairs`: entries 2i and 2i+1 turn together, else
     i and i + rot_dims/2; cos/sin scaled by mscale), then with `unit_norm`
-    every head is divided by its root mean square. Returns the new q; k and v (when given) go to the
-    paged caches."""
+    every head is divided by its root mean square. q_w / k_w [D]: every head
+    is divided by its root mean square and multiplied by them before the
+    turn. Returns the new q; k and v (when given) go to the paged caches."""
     T = q.shape[0]
 
-    def prep(z, n):
+    def prep(z, n, w):
         z = z.reshape(T, n, -1)
+        if w is not None:
+            z = rmsnorm(z.float(), w, eps)
         if rot_dims:
             z = rope_interleaved(z.float(), positions, inv_freq, mscale,
                                  rot_dims, pairs)
@@ -650,10 +654,11 @@ def rope_headnorm_store(q, k, v, positions, inv_freq, rot_dims, pairs,
         if unit_norm:
             z = z * torch.rsqrt(z.pow(2).mean(-1, keepdim=True) + eps)
         return z.reshape(T, -1)
-    store_paged(prep(k, kv_heads).to(k.dtype), k_cache, slot_mapping)
+    if k is not None:
+        store_paged(prep(k, kv_heads, k_w).to(k.dtype), k_cache, slot_mapping)
     if v is not None:
         store_paged(v, v_cache, slot_mapping)
-    return prep(q, heads).to(q.dtype)
+    return prep(q, heads, q_w).to(q.dtype)
 
 
 def polynorm(z, coef, eps):
@@ -732,3 +737,57 @@ def gelu_scaled(x, scale=None, ids=None, wts=None):
         scale = s.reshape(-1)
     s = 1.0 if scale is None else scale.view(*x.shape[:-1], 1)
     return F.gelu(x.float() * s).to(x.dtype)
+
+
+# ---------------------------------------------------------------------------
+# Retention (fixed decay per head, rotary positions, gated head norm), gate of
+# two row views. fp32 throughout.
+# ---------------------------------------------------------------------------
+def rope_table_rows(positions, inv_freq, mscale=1.0):
+    """fp32 [T, 2n]: cos | sin of position * frequency (fp64 angles)."""
+    a = positions.double()[:, None] * inv_freq.double()[None, :]
+    return torch.cat([torch.cos(a) * mscale, torch.sin(a) * mscale], -1).float()
+
+
+def retention(q, k, v, gate, table, k_scale, decay, state, slots, cu_q,
+              ctx_lens, eps):
+    """q, k [T, H*D] turned in the half layout by the rows of `table`, k times
+    k_scale; S_t = decay_h S_{t-1} + k_t v_t^T, o_t = S_t^T q_t; every head's o
+    divided by its root mean square, times silu(gate). state fp32 [slots, H, D,
+    Dv] in place; returns [T, H*Dv] in q's dtype."""
+    H, D, Dv = state.shape[1:]
+    T, rot = q.shape[0], table.shape[1]
+    half = rot // 2
+    cos, sin = table[:, None, :half], table[:, None, half:]
+
+    def turn(z):
+        z = z.float().reshape(T, H, D)
+        u, w = z[..., :half], z[..., half:rot]
+        return torch.cat([u * cos - w * sin, w * cos + u * sin, z[..., rot:]],
+                         -1)
+    qf, kf = turn(q), turn(k) * k_scale
+    vf = v.float().reshape(T, H, Dv)
+    a = decay[:, None, None]
+    o = torch.zeros(T, H, Dv, dtype=torch.float32)
+    for s, t0, t1 in _seq_ranges(T, slots, cu_q):
+        slot = int(slots[s])
+        if slot >= 0 and int(ctx_lens[s]) > 0:
+            S = state[slot].clone()
+        else:
+            S = torch.zeros(H, D, Dv, dtype=torch.float32)
+        for t in range(t0, t1):
+            S = a * S + kf[t][:, :, None] * vf[t][:, None, :]
+            o[t] = torch.einsum("hdv,hd->hv", S, qf[t])
+        if slot >= 0 and t1 > t0:
+            state[slot] = S
+    o = _unit_rms(o, eps).reshape(T, H * Dv)
+    return (o * F.silu(gate.float())).to(q.dtype)
+
+
+def glu_rows(g, u, gelu, row_gate=None):
+    """act(g) * u (* sigmoid(row_gate) [T, 1]), act = tanh GELU or SiLU."""
+    a = F.gelu(g.float(), approximate="tanh") if gelu else F.silu(g.float())
+    y = a * u.float()
+    if row_gate is not None:
+        y = y * torch.sigmoid(row_gate.float())
+    return y.to(g.dtype)
