@@ -21,6 +21,7 @@ from .scheduler import StepPlan
 from .sequence import Sequence
 
 BLOCK_SIZE = 16
+UNPAGED_BLOCKS = 1 << 20     # pool of a model without block-addressed caches
 
 
 class ModelRunner:
@@ -130,9 +131,10 @@ class ModelRunner:
         budget -= num_state_slots * sum(
             s.slot_bytes() for s in flat_specs(specs)
             if isinstance(s, (RecurrentState, ConvState)))
-        per_block = max(sum(s.block_bytes(BLOCK_SIZE, dtype_bytes)
-                            for s in specs), 1)
-        n = max(budget // per_block, 16)
+        per_block = sum(s.block_bytes(BLOCK_SIZE, dtype_bytes) for s in specs)
+        # nothing kept per token: blocks only count tokens, their number is
+        # free
+        n = max(budget // per_block, 16) if per_block else UNPAGED_BLOCKS
         if max_blocks:
             n = min(n, max_blocks)
         return int(n)
