@@ -98,7 +98,8 @@ def _tokens(cfg, n, seed):
 @functools.lru_cache(maxsize=None)
 def _oracle(name, tmp_root, n, seed):
     cfg, w, _ = _model(name, tmp_root)
-    return zo.forward(cfg, w, _tokens(cfg, n, seed))[0]
+    out, _, margin = zo.forward(cfg, w, _tokens(cfg, n, seed))
+    return out, margin
 
 
 def _engine(folder, target, blocks=64, slots=4, **kw):
@@ -110,8 +111,14 @@ def _engine(folder, target, blocks=64, slots=4, **kw):
 
 def _check(got, want, target, what=""):
     """fp32: every row close, but for a rare row where two experts' choice
-    scores nearly tie. bf16: rounding-sized error."""
-    e = rel_err(got, want)
+    scores nearly tie. bf16: rounding-sized error; rows whose choice hangs on
+    less than bf16 rounding of the router's input (want = (logits, choice
+    margins)) may differ."""
+    clear = slice(None)
+    if isinstance(want, tuple):
+        want, margin = want
+        clear = margin > (1e-5 if target[1] == torch.float32 else 0.01)
+    e = rel_err(got, want)[clear]
     if target[1] == torch.float32:
         assert float(e.median()) < 1e-4, (what, float(e.median()))
         assert int((e > 5e-4).sum()) <= len(e) // 40, (what, e)

@@ -154,10 +154,32 @@ def route(z, r):
     return [(e, s[e] * r.get("scale", 1.0)) for _, e in order[:r["top"]]]
 
 
-def ff_moe(h, w, f, mlp):
+def choice_margin(z, r):
+    """How clear the choice of one token is: the smallest score difference
+    between a kept and a dropped group, or a chosen and a passed-over expert
+    (infinite where nothing is dropped)."""
+    s = torch.sigmoid(z)
+    g = r.get("groups") or dict(count=1, keep=1)
+    s = s.view(g["count"], -1)
+    pair = s.topk(min(2, s.shape[1]), -1).values.sum(-1)
+    pair, order = pair.sort(descending=True)
+    gap = math.inf
+    if g["keep"] < g["count"]:
+        gap = float(pair[g["keep"] - 1] - pair[g["keep"]])
+    s = s[order[:g["keep"]]].reshape(-1).sort(descending=True).values
+    if len(s) > r["top"]:
+        gap = min(gap, float(s[r["top"] - 1] - s[r["top"]]))
+    return gap
+
+
+def ff_moe(h, w, f, mlp, margin=None):
+    """margin [T]: lowered to the tokens' choice margins."""
     out = torch.zeros_like(h)
     z = linear(h, w[f + "router"])
     for t in range(h.shape[0]):
+        if margin is not None:
+            margin[t] = min(float(margin[t]), choice_margin(z[t],
+                                                            mlp["router"]))
         for e, a in route(z[t], mlp["router"]):
             out[t] += a * expert(h[t:t + 1], w, f"{f}e{e}.")[0]
     if mlp.get("shared"):
@@ -168,13 +190,15 @@ def ff_moe(h, w, f, mlp):
 
 # ---- the stack --------------------------------------------------------------
 def forward(cfg, weights, tokens, dtype=torch.float64):
-    """-> (logits [T, vocab], residual after every layer [layers, T, W])."""
+    """-> (logits [T, vocab], residual after every layer [layers, T, W], choice
+    margin of every token over all routers [T])."""
     w = {k: (v.to(dtype) if v.is_floating_point() else v)
          for k, v in weights.items()}
     tokens = torch.as_tensor(tokens, dtype=torch.long)
     eps = cfg["norm"]["eps"]
     x = w["embed"][tokens] * (cfg.get("embedding") or {}).get("scale", 1.0)
     kept, after = {}, []
+    margin = torch.full((len(tokens),), math.inf)
     for i, lc in enumerate(cfg["layers"]):
         p, m = f"l{i}.", lc["mixer"]
         h = rms_norm(x, w[p + "norm1"], eps)
@@ -189,11 +213,11 @@ def forward(cfg, weights, tokens, dtype=torch.float64):
         mlp = lc.get("mlp")
         if mlp:
             y = y + (ff_dense(h, w, p + "mlp.") if mlp["kind"] == "dense"
-                     else ff_moe(h, w, p + "mlp.", mlp))
+                     else ff_moe(h, w, p + "mlp.", mlp, margin))
         x = x + y
         after.append(x)
     return linear(rms_norm(x, w["final.norm"], eps), w["head"]), \
-        torch.stack(after)
+        torch.stack(after), margin
 
 
 # ---- test models: configurations, random checkpoints, model folders ---------
