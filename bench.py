@@ -68,7 +68,7 @@ def parse_args():
     ap.add_argument("--hybrid-sizes", default="2k,4k")
     ap.add_argument("--hybrid-family", default="pugovik",
                     choices=("pugovik", "dunusun", "tosipel", "gararax",
-                             "nikedra"),
+                             "nikedra", "zokanex"),
                     help="which hybrid stack --mode hybrid measures beside "
                          "the equal-size llama stack")
     ap.add_argument("--model", default="llama-3-8b")
@@ -928,6 +928,189 @@ def _nikedra_kernels(size, device, T, batch, ctx):
     return out
 
 
+def _zokanex_kernels(size, device, T, batch, ctx):
+    """Achieved rates of the Zokanex kernels at one layer's shapes, each
+    beside the like kernel of the gararax / tosipel / pugovik / nikedra stacks
+    of that size. The results go into rows of the joint output operand, as in
+    the model."""
+    import torch.nn.functional as F
+    from xllm_service_amd.models.config import get_config
+    from xllm_service_amd.models.mixers import banded_rope_frequencies
+    from xllm_service_amd.ops import hybrid as hops
+    zc, tc, pc = (get_config(f"{f}-{size}") for f in (
+        "zokanex", "tosipel", "pugovik"))
+
+    def mixer(cfg, kind):
+        return next(l.mixer for l in cfg.layers if l.type == kind)
+    att, ret = mixer(zc, "attention"), mixer(zc, "retention")
+    tatt, lin = mixer(tc, "attention"), mixer(pc, "lightning")
+    dense = next(l.mlp for l in zc.layers if l.mlp["kind"] == "dense")
+    moe = next(l.mlp for l in zc.layers if l.mlp["kind"] == "moe")
+    bf = dict(dtype=torch.bfloat16, device=device)
+    f32 = dict(dtype=torch.float32, device=device)
+    i32 = dict(dtype=torch.int32, device=device)
+    out = []
+    nblk = (max(T, ctx) + 15) // 16
+    tab = torch.arange(batch * nblk, **i32).view(batch, nblk)
+    cu = torch.tensor([0, T], **i32)
+    sl = torch.tensor([T], **i32)
+    sld = torch.full((batch,), ctx, **i32)
+    z1 = torch.zeros(1, **i32)
+    sls = torch.arange(batch, **i32)
+    pos = torch.arange(T, dtype=torch.long, device=device)
+
+    def add(label, fn, work, unit, iters=20):
+        t = _time_gpu(fn, iters, 3)
+        scale = 1e12 if "FLOP" in unit else 1e6 if unit == "Mtok/s" else 1e9
+        out.append((label, t, work / t / scale, unit))
+    # ---- windowed attention ---------------------------------------------------
+    Wd, ff = zc.hidden_size, dense["ff"]
+    for label, m, joint in (("window attn", att, True),
+                            ("window+sink attn (tosipel)", tatt, False)):
+        H, G, D, Dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        win = m["mask"]["size"]
+        kc = torch.randn(batch * nblk, G, 16, D, **bf)
+        vc = torch.randn(batch * nblk, G, 16, Dv, **bf)
+        q = torch.randn(T, H * D, **bf)
+        o = torch.empty(T, H * Dv + ff, **bf)[:, :H * Dv] if joint \
+            else torch.empty(T, H, Dv, **f32)
+        kw = dict(window=win,
+                  sink=None if joint else torch.zeros(H, **f32))
+        seen = sum(min(i + 1, win) for i in range(T))
+        add(f"{label} prefill ({win})",
+            lambda: hops.capped_attn(q, kc, vc, tab[:1], cu, sl, H,
+                                     m["scale"], 0.0, o, **kw),
+            2.0 * H * (D + Dv) * seen, "TFLOP/s", 5)
+        add(f"{label} decode ({win})",
+            lambda: hops.capped_attn(q[:batch], kc, vc, tab, None, sld, H,
+                                     m["scale"], 0.0, o[:batch], **kw),
+            batch * min(ctx, win) * G * (D + Dv) * 2, "GB/s")
+        del kc, vc
+    # ---- retention vs decayed linear attention ----------------------------------
+    H, D, Dv, rot = ret["heads"], ret["dim"], ret["vdim"], ret["rot"]
+    a, b = H * D, H * Dv
+    p = torch.randn(T, 2 * a + 2 * b, **bf)
+    dec = torch.tensor(ret["decay"], **f32)
+    st = torch.zeros(batch, H, D, Dv, **f32)
+    y = torch.empty(T, b + ff, **bf)
+    inv = banded_rope_frequencies(rot).to(device)
+    table = hops.rope_table(pos, inv)
+    tokens = ((T, z1, cu, z1, "prefill"), (batch, sls, None, sld, "decode"))
+    for n, slots, cuq, ctxl, tail in tokens:
+        q, k, v, g = (p[:n, i:j] for i, j in (
+            (0, a), (a, 2 * a), (2 * a, 2 * a + b), (2 * a + b, 2 * a + 2 * b)))
+        add(f"retention + norm + gate {tail}",
+            lambda: hops.retention(q, k, v, g, table[:n], D ** -0.5, dec, st,
+                                   slots, cuq, ctxl, 1e-6, y[:n, :b]),
+            4.0 * H * D * Dv * T if cuq is not None
+            else batch * H * D * Dv * 8,
+            "GB/s" if cuq is None else "TFLOP/s (recurrence form)")
+    Hp, Dp, Vp = lin["heads"], lin["dim"], lin["vdim"]
+    pl = torch.randn(T, 2 * Hp * Dp + Hp * Vp, **bf)
+    decp = torch.tensor(lin["decay"], **f32)
+    stp = torch.zeros(batch, Hp, Dp, Vp, **f32)
+    op = torch.empty(T, Hp, Vp, **f32)
+    for n, slots, cuq, ctxl, tail in tokens:
+        q, k, v = pl[:n, :Hp * Dp], pl[:n, Hp * Dp:2 * Hp * Dp], \
+            pl[:n, 2 * Hp * Dp:]
+        add(f"decay_attn (pugovik) {tail}",
+            lambda: hops.decay_attn(q, k, v, decp, stp, slots, cuq, ctxl,
+                                    op[:n], max_q_len=n),
+            4.0 * Hp * Dp * Vp * T if cuq is not None
+            else batch * Hp * Dp * Vp * 8,
+            "GB/s" if cuq is None else "TFLOP/s (recurrence form)", 5)
+    add("rope_table", lambda: hops.rope_table(pos, inv), T * rot["dims"] * 4,
+        "GB/s")
+    # ---- query/key preparation --------------------------------------------------
+    H, G, D, Dv = att["heads"], att["kv_heads"], att["dim"], att["vdim"]
+    rd = att["rot"]["dims"]
+    proj = torch.randn(T, H * D + G * D + G * Dv, **bf)
+    kc = torch.zeros(nblk, G, 16, D, **bf)
+    vc = torch.zeros(nblk, G, 16, Dv, **bf)
+    w = torch.ones(D, **f32)
+    wq, wk = torch.ones(H * D, **f32), torch.ones(G * D, **f32)
+    inv = banded_rope_frequencies(att["rot"]).to(device)
+    table = hops.rope_table(pos, inv)
+    q, k, v = proj[:, :H * D], proj[:, H * D:H * D + G * D], \
+        proj[:, H * D + G * D:]
+    nb = T * (2 * H * D + 2 * G * D + 2 * G * Dv) * 2
+    args = (pos, inv, rd, False, False, 1e-6, H, G, kc, vc, pos, 1.0)
+    add("head norm + turn + store",
+        lambda: hops.rope_headnorm_store(q, k, v, *args, w, w, table), nb,
+        "GB/s")
+    add("head norm + turn, borrowed keys",
+        lambda: hops.rope_headnorm_store(q, None, None, *args, w, None, table),
+        T * 2 * H * D * 2, "GB/s")
+    add("rope_headnorm_store (gararax)",
+        lambda: hops.rope_headnorm_store(
+            q, k, v, pos, inv, rd, True, True, 1e-6, H, G, kc, vc, pos), nb,
+        "GB/s")
+    add("rownorm_rope_store (tosipel)",
+        lambda: hops.rownorm_rope_store(q, k, v, wq, wk, 1e-6, pos, inv, rd,
+                                        H, G, kc, vc, pos), nb, "GB/s")
+    # ---- residual ---------------------------------------------------------------
+    x, wn = torch.randn(T, Wd, **f32), torch.ones(Wd, **f32)
+    top = moe["router"]["top"]
+    ya = torch.randn(T, Wd, **bf)
+    ye = torch.randn(T * top, Wd, **bf)
+    rows = torch.randperm(T * top, device=device).to(torch.int32) \
+        .view(T, top)
+    wts = torch.rand(T, top, **f32)
+    hist, one = torch.randn(2, T, Wd, **f32), torch.ones(1, **f32)
+    for n, tail in ((T, ""), (batch, f", {batch} rows (decode)")):
+        xn, yn = x[:n], ya[:n]
+        add(f"join_norm{tail}",
+            lambda: hops.join_norm_(xn, yn, None, wn, 1e-6), n * Wd * 12,
+            "GB/s")
+        rn = rows[:n] % (n * top)
+        add(f"join_norm + experts{tail}",
+            lambda: hops.join_norm_(xn, yn, (ye, rn, wts[:n]), wn, 1e-6),
+            n * Wd * (12 + 2 * top), "GB/s")
+        hn = hist[:, :n].contiguous()
+        add(f"depth_mix_norm level 1 (nikedra){tail}",
+            lambda: hops.depth_mix_norm(
+                hn[0], hn, 1, yn, None, None, None, 1.0, yn, one.expand(2)
+                .contiguous(), one, None, 1e-6, torch.bfloat16, xn),
+            n * Wd * 20, "GB/s")
+        add(f"norm_residual_add + next norm (gararax){tail}",
+            lambda: hops.norm_residual_add_(xn, yn, wn, 1e-6, torch.bfloat16,
+                                            wn), n * Wd * 12, "GB/s")
+    add("moe_combine (pugovik)", lambda: hops.moe_combine(ye, rows, wts, T),
+        T * Wd * (2 * top + 4), "GB/s")
+    # ---- gates ------------------------------------------------------------------
+    gu = torch.randn(T, 2 * ff + 16, **bf)
+    yo = torch.empty(T, Wd + ff, **bf)
+    add("glu_rows gelu", lambda: hops.glu_rows(
+        gu[:, :ff], gu[:, ff:2 * ff], yo[:, Wd:], gelu=True), T * ff * 6,
+        "GB/s")
+    sf = moe["shared"]["ff"]
+    add("glu_rows silu + row gate", lambda: hops.glu_rows(
+        gu[:, :sf], gu[:, sf:2 * sf], yo[:, Wd:Wd + sf], gelu=False,
+        row_gate=gu[:, 2 * sf:2 * sf + 1]), T * sf * 6, "GB/s")
+    g2 = torch.randn(T, 2 * ff, **bf)
+    add("gelu_tanh_mul (tosipel)", lambda: hops.gelu_tanh_mul(g2), T * ff * 6,
+        "GB/s")
+    # ---- router -----------------------------------------------------------------
+    r = moe["router"]
+    h, wr = torch.randn(T, Wd, **bf), torch.randn(r["experts"], Wd, **f32)
+    gr = r["groups"]
+    add("moe_route with scale", lambda: hops.moe_route(
+        h, wr, r["top"], gr["count"], gr["keep"], scale=r["scale"]), T,
+        "Mtok/s")
+    # ---- one output GEMM for mixer and feed-forward vs two ------------------------
+    wo, wd = torch.randn(Wd, Wd, **bf), torch.randn(Wd, ff, **bf)
+    wj = torch.cat([wo, wd], 1).contiguous()
+    for n, tail in ((T, "prefill"), (batch, f"{batch} rows")):
+        yj = torch.randn(n, Wd + ff, **bf)
+        y1, y2 = yj[:, :Wd].contiguous(), yj[:, Wd:].contiguous()
+        fl = 2.0 * n * Wd * (Wd + ff)
+        add(f"joint output GEMM, {tail}", lambda: F.linear(yj, wj), fl,
+            "TFLOP/s")
+        add(f"two output GEMMs, {tail}",
+            lambda: (F.linear(y1, wo), F.linear(y2, wd)), fl, "TFLOP/s")
+    return out
+
+
 def run_hybrid_mode(args, device):
     assert torch.cuda.is_available(), "hybrid mode measures the HIP path"
     kernels = _hybrid_kernels
@@ -944,6 +1127,9 @@ def run_hybrid_mode(args, device):
     if args.hybrid_family == "nikedra":
         kernels = _nikedra_kernels
         fams = ("nikedra", "tosipel", "dunusun", "pugovik", "llama")
+    if args.hybrid_family == "zokanex":
+        kernels = _zokanex_kernels
+        fams = ("zokanex", "gararax", "pugovik", "nikedra", "llama")
     for size in args.hybrid_sizes.split(","):
         T, batch, ctx = 4096, 32, 2048
         for name, t, rate, unit in kernels(size, device, T, batch, ctx):

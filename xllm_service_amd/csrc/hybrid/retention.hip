@@ -31,8 +31,11 @@
 // The order in which the contraction index is walked is free as long as A and
 // B agree. Pass 2 forms S^T = K Q^T, so that a lane's four scores are the
 // keys g*4 .. g*4+3 of ONE query, which is what the B operand of
-// O^T += V^T P^T wants of that lane: no exchange between lanes. Output
-// columns of a query end up as four neighbours per lane and column tile.
+// O^T += V^T P^T wants of that lane: no exchange between lanes. Which value
+// column a row of the transposed product stands for is free too: row m of
+// product j is column (j / 4) * 64 + m * 4 + j % 4, so a lane fetches the
+// operands of four products with one 16 B read and ends up with four
+// neighbouring output columns. The key rows of pass 1 are dealt the same way.
 #include "hybrid_common.h"
 
 namespace xllm {
@@ -43,35 +46,42 @@ typedef __attribute__((__vector_size__(4 * sizeof(float)))) float f32x4;
 constexpr int RT_C = 64;       // tokens per chunk
 constexpr int RT_S = 32;       // tokens staged per LDS fill
 
-// one operand of q/k/v rows of a head: T rows with a stride, D columns
+// q, k or v rows of a head: stride, columns
 template <typename T>
 struct RTRows {
-  const T* p; long stride; int width; int vec;    // vec: quads are aligned
+  const T* p; long stride; int width;
 };
 struct RTRot {
   const float* cs; int rot;                       // table [tokens, rot]
 };
 
-// columns c .. c+3 of a row, turned; zeros beyond the width
-template <typename T>
-XLLM_DEV void rt_load4(const T* row, int c, int width, int vec,
-                       const float* cs, int rot, float v[4]) {
+// Columns c .. c+3 of a row, turned; zeros beyond the width. VEC: widths,
+// strides and rot/2 are multiples of four and quads are aligned; addresses are
+// clamped instead of branching, so that several of these loads can be in flight
+// together.
+template <typename T, bool VEC>
+XLLM_DEV void rt_load4(const T* row, int c, int width, const float* cs,
+                       int rot, float v[4]) {
   const int half = rot >> 1;
-  if (vec) {
-    if (c >= width) { v[0] = v[1] = v[2] = v[3] = 0.f; return; }
-    Quad<T>::ld(row + c, v);
-    if (c < rot) {                                // vec: rot/2 % 4 == 0
-      const bool first = c < half;
-      const int i = first ? c : c - half;
+  if (VEC) {
+    const bool in = c < width;
+    Quad<T>::ld(row + (in ? c : 0), v);
+    if (rot > 0) {                                // uniform; rot/2 % 4 == 0
+      const bool turned = c < rot, first = c < half;
+      const int i = turned ? (first ? c : c - half) : 0;
       float y[4], co[4], si[4];
-      Quad<T>::ld(row + (first ? c + half : c - half), y);
+      Quad<T>::ld(row + (first ? i + half : i), y);
       Quad<float>::ld(cs + i, co);
       Quad<float>::ld(cs + half + i, si);
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        v[j] = first ? v[j] * co[j] - y[j] * si[j]
-                     : v[j] * co[j] + y[j] * si[j];
+      for (int j = 0; j < 4; ++j) {
+        const float z = first ? v[j] * co[j] - y[j] * si[j]
+                              : v[j] * co[j] + y[j] * si[j];
+        v[j] = turned ? z : v[j];
+      }
     }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = in ? v[j] : 0.f;
     return;
   }
 #pragma unroll
@@ -91,23 +101,32 @@ XLLM_DEV void rt_load4(const T* row, int c, int width, int vec,
   }
 }
 
-// RT_S rows into dst [RT_S][WP + 4], row r times mul[r] (or one number)
-template <typename T, int WP>
+// RT_S rows into dst [RT_S][WP + 4], row r times mul (and pw[last - r]); rows
+// past `rows` (>= 1) become zeros. B quads per thread are fetched together.
+template <typename T, int WP, int B, bool VEC>
 XLLM_DEV void rt_stage(float* dst, const RTRows<T>& R, long row0, int rows,
                        const RTRot& rot, float mul, const float* pw, int last) {
-  for (int idx = threadIdx.x; idx < RT_S * (WP / 4); idx += 256) {
-    const int r = idx / (WP / 4), c = (idx - r * (WP / 4)) * 4;
-    float v[4] = {0.f, 0.f, 0.f, 0.f};
-    if (r < rows) {
-      const long t = row0 + r;
-      rt_load4<T>(R.p + t * R.stride, c, R.width, R.vec,
-                  rot.cs + t * rot.rot, rot.rot, v);
-      const float m = pw != nullptr ? mul * pw[last - r] : mul;
+  constexpr int N = RT_S * (WP / 4) / 256;        // quads per thread
+  static_assert(N % B == 0, "whole batches");
+#pragma unroll 1
+  for (int b = 0; b < N; b += B) {
+    float v[B][4];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) v[j] *= m;
+    for (int i = 0; i < B; ++i) {
+      const int idx = threadIdx.x + (b + i) * 256;
+      const int r = idx / (WP / 4), c = (idx - r * (WP / 4)) * 4;
+      const long t = row0 + min(r, rows - 1);
+      rt_load4<T, VEC>(R.p + t * R.stride, c, R.width, rot.cs + t * rot.rot,
+                       rot.rot, v[i]);
     }
-    *reinterpret_cast<float4*>(dst + r * (WP + 4) + c) =
-        make_float4(v[0], v[1], v[2], v[3]);
+#pragma unroll
+    for (int i = 0; i < B; ++i) {
+      const int idx = threadIdx.x + (b + i) * 256;
+      const int r = idx / (WP / 4), c = (idx - r * (WP / 4)) * 4;
+      const float m = r >= rows ? 0.f : pw != nullptr ? mul * pw[last - r] : mul;
+      *reinterpret_cast<float4*>(dst + r * (WP + 4) + c) =
+          make_float4(v[i][0] * m, v[i][1] * m, v[i][2] * m, v[i][3] * m);
+    }
   }
 }
 
@@ -132,8 +151,9 @@ XLLM_DEV bool rt_locate(int b, const int* cu_q, int n_seqs, int* s, int* c,
 // ---- pass 1: what a chunk adds to the state -----------------------------------
 // ws [chunks][H][D][Dv]; DP, VP: widths padded to the tile grid; blockIdx.z
 // is the block of VP value columns
-template <typename T, int DP, int VP>
-__global__ void __launch_bounds__(256) retention_sum_kernel(
+template <typename T, int DP, int VP, bool VEC>
+__global__ void
+__launch_bounds__(256, DP == 256 ? 2 : 4) retention_sum_kernel(
     float* __restrict__ ws, RTRows<T> K, RTRows<T> V, RTRot rot, float k_scale,
     const float* __restrict__ decay, const int* __restrict__ cu_q, int n_seqs,
     int heads, int D, int Dv) {
@@ -163,24 +183,25 @@ __global__ void __launch_bounds__(256) retention_sum_kernel(
   for (int b0 = 0; b0 < len; b0 += RT_S) {
     const int nt = min(RT_S, len - b0);
     if (b0) __syncthreads();
-    rt_stage<T, DP>(ks, K, t0 + b0, nt, rot, k_scale, pw, len - 1 - b0);
-    rt_stage<T, VP>(vs, V, t0 + b0, nt, none, 1.0f, nullptr, 0);
+    rt_stage<T, DP, 2, VEC>(ks, K, t0 + b0, nt, rot, k_scale, pw, len - 1 - b0);
+    rt_stage<T, VP, 2, VEC>(vs, V, t0 + b0, nt, none, 1.0f, nullptr, 0);
     __syncthreads();
 #pragma unroll
     for (int st = 0; st < RT_S / 4; ++st) {
-      const float* kr = ks + (st * 4 + g) * LK + w * DT * 16 + n;
-      const float* vr = vs + (st * 4 + g) * LV + n;
+      const float* kr = ks + (st * 4 + g) * LK + w * DT * 16 + n * DT;
+      const float* vr = vs + (st * 4 + g) * LV + n * 4;
       float a[DT];
 #pragma unroll
-      for (int i = 0; i < DT; ++i) a[i] = kr[i * 16];
+      for (int i = 0; i < DT; ++i) a[i] = kr[i];
+      float b[VT];
 #pragma unroll
-      for (int j = 0; j < VT; ++j) {
-        const float b = vr[j * 16];
+      for (int j = 0; j < VT; j += 4) Quad<float>::ld(vr + j * 16, b + j);
+#pragma unroll
+      for (int j = 0; j < VT; ++j)
 #pragma unroll
         for (int i = 0; i < DT; ++i)
-          acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], b, acc[i][j],
-                                                           0, 0, 0);
-      }
+          acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+              a[i], b[j], acc[i][j], 0, 0, 0);
     }
   }
   float* dst = ws + ((long)blockIdx.x * heads + h) * D * (long)Dv + v0;
@@ -188,11 +209,21 @@ __global__ void __launch_bounds__(256) retention_sum_kernel(
   for (int i = 0; i < DT; ++i)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int d = (w * DT + i) * 16 + g * 4 + r;
+      const int d = w * DT * 16 + (g * 4 + r) * DT + i;
+      if (d >= D) continue;
 #pragma unroll
-      for (int j = 0; j < VT; ++j) {
-        const int col = j * 16 + n;
-        if (d < D && col < V.width) dst[(long)d * Dv + col] = acc[i][j][r];
+      for (int j = 0; j < VT; j += 4) {
+        const int col = j * 16 + n * 4, left = V.width - col;
+        float* p = dst + (long)d * Dv + col;
+        const float x[4] = {acc[i][j][r], acc[i][j + 1][r], acc[i][j + 2][r],
+                            acc[i][j + 3][r]};
+        if (VEC) {
+          if (left > 0) Quad<float>::st(p, x);
+        } else {
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            if (e < left) p[e] = x[e];
+        }
       }
     }
 }
@@ -246,10 +277,10 @@ __global__ void retention_scan_kernel(float* __restrict__ ws,
 }
 
 // four neighbouring outputs of one head, normed and gated
-template <typename T>
-XLLM_DEV void rt_store4(T* dst, const T* gate, const f32x4& o, float rs, int n,
-                        int vec) {
-  if (vec) {
+template <typename T, bool VEC>
+XLLM_DEV void rt_store4(T* dst, const T* gate, const f32x4& o, float rs,
+                        int n) {
+  if (VEC) {
     float gv[4], y[4];
     Quad<T>::ld(gate, gv);
 #pragma unroll
@@ -264,11 +295,12 @@ XLLM_DEV void rt_store4(T* dst, const T* gate, const f32x4& o, float rs, int n,
 
 // ---- pass 2: the outputs of a chunk ---------------------------------------------
 // FUSED (all value columns in one workgroup): y into `out` rows; else the
-// plain o into fp32 o_raw [T, H, Dv].
-template <typename T, int DP, int VP, bool FUSED>
-__global__ void __launch_bounds__(256) retention_out_kernel(
+// plain o into fp32 o_raw [T, H, Dv]. The launch bound keeps the accumulators
+// in plain registers (three to four waves per SIMD, no spills).
+template <typename T, int DP, int VP, bool FUSED, bool VEC>
+__global__ void __launch_bounds__(256, 3) retention_out_kernel(
     T* __restrict__ out, long out_stride, float* __restrict__ o_raw,
-    const T* __restrict__ gate, long gate_stride, int out_vec, float eps,
+    const T* __restrict__ gate, long gate_stride, float eps,
     const float* __restrict__ ws, RTRows<T> Q, RTRows<T> K, RTRows<T> V,
     RTRot rot, float k_scale, const float* __restrict__ decay,
     const int* __restrict__ slots, const int* __restrict__ cu_q,
@@ -302,8 +334,8 @@ __global__ void __launch_bounds__(256) retention_out_kernel(
     qv[i][0] = qv[i][1] = qv[i][2] = qv[i][3] = 0.f;
     if (q_ok) {
       const long t = t0 + qi;
-      rt_load4<T>(Q.p + t * Q.stride, i * 16 + g * 4, Q.width, Q.vec,
-                  rot.cs + t * rot.rot, rot.rot, qv[i]);
+      rt_load4<T, VEC>(Q.p + t * Q.stride, i * 16 + g * 4, Q.width,
+                       rot.cs + t * rot.rot, rot.rot, qv[i]);
     }
   }
   f32x4 acc[VT];
@@ -313,10 +345,10 @@ __global__ void __launch_bounds__(256) retention_out_kernel(
   // ---- within the chunk ---------------------------------------------------------
   for (int b0 = 0; b0 < len; b0 += RT_S) {
     __syncthreads();
-    rt_stage<T, DP>(ks, K, t0 + b0, min(RT_S, len - b0), rot, k_scale, nullptr,
-                    0);
-    rt_stage<T, VP>(vs, V, t0 + b0, min(RT_S, len - b0), none, 1.0f, nullptr,
-                    0);
+    rt_stage<T, DP, 2, VEC>(ks, K, t0 + b0, min(RT_S, len - b0), rot, k_scale,
+                       nullptr, 0);
+    rt_stage<T, VP, VP / 32, VEC>(vs, V, t0 + b0, min(RT_S, len - b0), none, 1.0f,
+                             nullptr, 0);
     __syncthreads();
     if (!wave_on) continue;
 #pragma unroll
@@ -338,11 +370,14 @@ __global__ void __launch_bounds__(256) retention_out_kernel(
       for (int r = 0; r < 4; ++r) {
         const int back = qi - (kb + g * 4 + r);
         const float p = back >= 0 ? (p0[r] + p1[r]) * pw[back] : 0.f;
-        const float* vr = vs + (kt * 16 + g * 4 + r) * LV + n;
+        const float* vr = vs + (kt * 16 + g * 4 + r) * LV + n * 4;
+        float a[VT];
+#pragma unroll
+        for (int j = 0; j < VT; j += 4) Quad<float>::ld(vr + j * 16, a + j);
 #pragma unroll
         for (int j = 0; j < VT; ++j)
-          acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(vr[j * 16], p, acc[j],
-                                                        0, 0, 0);
+          acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[j], p, acc[j], 0, 0,
+                                                        0);
       }
     }
   }
@@ -353,22 +388,30 @@ __global__ void __launch_bounds__(256) retention_out_kernel(
 #pragma unroll
     for (int sl = 0; sl < DP / 64; ++sl) {
       __syncthreads();
-      for (int idx = tid; idx < 64 * (VP / 4); idx += 256) {
-        const int d = idx / (VP / 4), cc = (idx - d * (VP / 4)) * 4;
-        const int dd = sl * 64 + d;
-        float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
-        if (dd < D) {
-          const float* p = S + (long)dd * Dv + cc;
-          if ((Dv & 3) == 0 && cc < V.width) {
-            x = *reinterpret_cast<const float4*>(p);
-          } else {
-            if (cc < V.width) x.x = p[0];
-            if (cc + 1 < V.width) x.y = p[1];
-            if (cc + 2 < V.width) x.z = p[2];
-            if (cc + 3 < V.width) x.w = p[3];
-          }
+      constexpr int NS = 64 * (VP / 4) / 256;         // quads per thread
+      float4 x[NS];
+#pragma unroll
+      for (int i = 0; i < NS; ++i) {
+        const int idx = tid + i * 256;
+        const int d = sl * 64 + idx / (VP / 4), cc = idx % (VP / 4) * 4;
+        const float* p = S + (long)min(d, D - 1) * Dv;
+        if (VEC) {
+          x[i] = *reinterpret_cast<const float4*>(p + (cc < V.width ? cc : 0));
+        } else {
+          const int e = V.width - 1;
+          x[i] = make_float4(p[min(cc, e)], p[min(cc + 1, e)],
+                             p[min(cc + 2, e)], p[min(cc + 3, e)]);
         }
-        *reinterpret_cast<float4*>(ss + d * LV + cc) = x;
+      }
+#pragma unroll
+      for (int i = 0; i < NS; ++i) {
+        const int idx = tid + i * 256;
+        const int d = idx / (VP / 4), cc = idx % (VP / 4) * 4;
+        const bool in = sl * 64 + d < D;
+        const int left = in ? V.width - cc : 0;       // columns that exist
+        *reinterpret_cast<float4*>(ss + d * LV + cc) =
+            make_float4(left > 0 ? x[i].x : 0.f, left > 1 ? x[i].y : 0.f,
+                        left > 2 ? x[i].z : 0.f, left > 3 ? x[i].w : 0.f);
       }
       __syncthreads();
       if (!wave_on) continue;
@@ -377,15 +420,18 @@ __global__ void __launch_bounds__(256) retention_out_kernel(
 #pragma unroll
         for (int q4 = 0; q4 < 4; ++q4) {
           const float b = qv[sl * 4 + i][q4] * fade;
-          const float* sr = ss + (i * 16 + g * 4 + q4) * LV + n;
+          const float* sr = ss + (i * 16 + g * 4 + q4) * LV + n * 4;
+          float a[VT];
+#pragma unroll
+          for (int j = 0; j < VT; j += 4) Quad<float>::ld(sr + j * 16, a + j);
 #pragma unroll
           for (int j = 0; j < VT; ++j)
-            acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(sr[j * 16], b,
-                                                          acc[j], 0, 0, 0);
+            acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[j], b, acc[j], 0,
+                                                          0, 0);
         }
     }
   }
-  // acc[j][r] = o[query qi][column v0 + j*16 + g*4 + r]
+  // acc[j][r] = o[query qi][column v0 + (j/4)*64 + (g*4 + r)*4 + j%4]
   float sq = 0.f;
   if (FUSED) {
 #pragma unroll
@@ -402,18 +448,22 @@ __global__ void __launch_bounds__(256) retention_out_kernel(
     T* orow = out + t * out_stride + (long)h * Dv;
     const T* grow = gate + t * gate_stride + (long)h * Dv;
 #pragma unroll
-    for (int j = 0; j < VT; ++j) {
-      const int col = j * 16 + g * 4;
-      if (col < Dv)
-        rt_store4<T>(orow + col, grow + col, acc[j], rs, Dv - col, out_vec);
-    }
+    for (int j = 0; j < VT; j += 4)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int col = j * 16 + (g * 4 + r) * 4;
+        const f32x4 o = {acc[j][r], acc[j + 1][r], acc[j + 2][r],
+                         acc[j + 3][r]};
+        if (col < Dv)
+          rt_store4<T, VEC>(orow + col, grow + col, o, rs, Dv - col);
+      }
   } else {
     float* orow = o_raw + (t * heads + h) * (long)Dv + v0;
 #pragma unroll
     for (int j = 0; j < VT; ++j)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const int col = j * 16 + g * 4 + r;
+        const int col = (j & ~3) * 16 + (g * 4 + r) * 4 + (j & 3);
         if (col < V.width) orow[col] = acc[j][r];
       }
   }
@@ -545,37 +595,33 @@ long retention_chunks(long tokens, long n_seqs) {
 // value columns one workgroup of pass 2 holds: the fused form needs all
 int retention_fused_columns() { return 128; }
 
-template <typename T, int DP, int VP>
+template <typename T, int DP, int VP, bool VEC>
 static void rt_prefill(T* out, long out_stride, float* o_raw, const T* gate,
-                       long gate_stride, int out_vec, float eps, float* ws,
-                       RTRows<T> Q, RTRows<T> K, RTRows<T> V, RTRot rot,
-                       float k_scale, const float* decay, float* state,
-                       const int* slots, const int* cu_q, const int* ctx_lens,
-                       long tokens, int n_seqs, int heads, int D, int Dv,
-                       hipStream_t st) {
+                       long gate_stride, float eps, float* ws, RTRows<T> Q,
+                       RTRows<T> K, RTRows<T> V, RTRot rot, float k_scale,
+                       const float* decay, float* state, const int* slots,
+                       const int* cu_q, const int* ctx_lens, long tokens,
+                       int n_seqs, int heads, int D, int Dv, hipStream_t st) {
   const dim3 grid((unsigned)retention_chunks(tokens, n_seqs), heads,
                   (Dv + VP - 1) / VP);
   const size_t lds = (size_t)RT_S * (DP + 4 + VP + 4) * sizeof(float);
   const size_t lds2 = lds > (size_t)64 * (VP + 4) * sizeof(float)
       ? lds : (size_t)64 * (VP + 4) * sizeof(float);
-  hipLaunchKernelGGL((retention_sum_kernel<T, DP, VP>), grid, dim3(256), lds,
-                     st, ws, K, V, rot, k_scale, decay, cu_q, n_seqs, heads, D,
-                     Dv);
+  hipLaunchKernelGGL((retention_sum_kernel<T, DP, VP, VEC>), grid, dim3(256),
+                     lds, st, ws, K, V, rot, k_scale, decay, cu_q, n_seqs,
+                     heads, D, Dv);
   const long per_head = (long)D * Dv, per_seq = per_head * heads;
   hipLaunchKernelGGL(retention_scan_kernel,
                      dim3((unsigned)((per_seq + 255) / 256), n_seqs),
                      dim3(256), 0, st, ws, state, decay, slots, cu_q, ctx_lens,
                      heads, per_head);
-  if (o_raw == nullptr)
-    hipLaunchKernelGGL((retention_out_kernel<T, DP, VP, true>), grid,
-                       dim3(256), lds2, st, out, out_stride, o_raw, gate,
-                       gate_stride, out_vec, eps, ws, Q, K, V, rot, k_scale,
-                       decay, slots, cu_q, ctx_lens, n_seqs, heads, D, Dv);
-  else
-    hipLaunchKernelGGL((retention_out_kernel<T, DP, VP, false>), grid,
-                       dim3(256), lds2, st, out, out_stride, o_raw, gate,
-                       gate_stride, out_vec, eps, ws, Q, K, V, rot, k_scale,
-                       decay, slots, cu_q, ctx_lens, n_seqs, heads, D, Dv);
+#define RT_OUT(FUSED)                                                         \
+  hipLaunchKernelGGL((retention_out_kernel<T, DP, VP, FUSED, VEC>), grid,     \
+                     dim3(256), lds2, st, out, out_stride, o_raw, gate,       \
+                     gate_stride, eps, ws, Q, K, V, rot, k_scale, decay,      \
+                     slots, cu_q, ctx_lens, n_seqs, heads, D, Dv)
+  if (o_raw == nullptr) RT_OUT(true); else RT_OUT(false);
+#undef RT_OUT
 }
 
 // cu_q == nullptr: decode rows (ws and o_raw unused). o_raw != nullptr: plain
@@ -590,16 +636,8 @@ void launch_retention(T* out, long out_stride, float* o_raw, const T* gate,
                       long tokens, int n_seqs, int heads, int D, int Dv,
                       hipStream_t st) {
   if (n_seqs == 0 || tokens == 0) return;
-  const int q4 = 4 * (int)sizeof(T) - 1;          // alignment of a quad
-  auto quads = [&](const T* p, long stride, int width) {
-    return width % 4 == 0 && stride % 4 == 0 &&
-           (reinterpret_cast<uintptr_t>(p) & q4) == 0;
-  };
-  const int rot_ok = rot_dims % 8 == 0 &&
-                     (reinterpret_cast<uintptr_t>(cs) & 15) == 0;
-  RTRows<T> Q = {q, q_stride, D, quads(q, q_stride, D) && rot_ok};
-  RTRows<T> K = {k, k_stride, D, quads(k, k_stride, D) && rot_ok};
-  RTRows<T> V = {v, v_stride, Dv, quads(v, v_stride, Dv)};
+  const RTRows<T> Q = {q, q_stride, D}, K = {k, k_stride, D},
+                  V = {v, v_stride, Dv};
   const RTRot rot = {cs, rot_dims};
   if (cu_q == nullptr) {
     const int vec = Dv % 4 == 0 ? 4 : 1;
@@ -618,15 +656,24 @@ void launch_retention(T* out, long out_stride, float* o_raw, const T* gate,
                          slots, ctx_lens, heads, D, Dv);
     return;
   }
-  const int out_vec = quads(out, out_stride, Dv) &&
-                      quads(gate, gate_stride, Dv);
-#define RT_CALL(DP, VP)                                                       \
-  rt_prefill<T, DP, VP>(out, out_stride, o_raw, gate, gate_stride, out_vec,   \
-                        eps, ws, Q, K, V, rot, k_scale, decay, state, slots,  \
-                        cu_q, ctx_lens, tokens, n_seqs, heads, D, Dv, st)
-  if (D <= 64) { if (Dv <= 64) RT_CALL(64, 64); else RT_CALL(64, 128); }
-  else if (D <= 128) { if (Dv <= 64) RT_CALL(128, 64); else RT_CALL(128, 128); }
-  else { if (Dv <= 64) RT_CALL(256, 64); else RT_CALL(256, 128); }
+  auto quads = [](const void* p, long stride, size_t size) {
+    return stride % 4 == 0 &&
+           reinterpret_cast<uintptr_t>(p) % (4 * size) == 0;
+  };
+  const bool vec = D % 4 == 0 && Dv % 4 == 0 && rot_dims % 8 == 0 &&
+                   quads(cs, rot_dims, 4) && quads(q, q_stride, sizeof(T)) &&
+                   quads(k, k_stride, sizeof(T)) &&
+                   quads(v, v_stride, sizeof(T)) &&
+                   quads(gate, gate_stride, sizeof(T)) &&
+                   quads(out, out_stride, sizeof(T));
+#define RT_CALL(DP, VP, VEC)                                                  \
+  rt_prefill<T, DP, VP, VEC>(out, out_stride, o_raw, gate, gate_stride, eps,  \
+                             ws, Q, K, V, rot, k_scale, decay, state, slots,  \
+                             cu_q, ctx_lens, tokens, n_seqs, heads, D, Dv, st)
+  if (!vec) RT_CALL(256, 128, false);     // odd widths: one size for all
+  else if (D <= 64) { if (Dv <= 64) RT_CALL(64, 64, true); else RT_CALL(64, 128, true); }
+  else if (D <= 128) { if (Dv <= 64) RT_CALL(128, 64, true); else RT_CALL(128, 128, true); }
+  else { if (Dv <= 64) RT_CALL(256, 64, true); else RT_CALL(256, 128, true); }
 #undef RT_CALL
 }
 

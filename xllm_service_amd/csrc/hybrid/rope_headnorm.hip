@@ -114,6 +114,105 @@ __global__ void __launch_bounds__(256) rope_headnorm_store_kernel(
   }
 }
 
+// The same with four neighbouring entries per lane: LG lanes own a head, 256 /
+// LG heads are prepared side by side, and the entry a turned one is paired
+// with comes from a lane of the same group (or, with `pairs`, from the same
+// quad) instead of a second read. D, rot/2 and the row strides are multiples
+// of four, D <= 4 * LG.
+template <typename T, int LG>
+__global__ void __launch_bounds__(256) rope_headnorm_quads_kernel(
+    T* __restrict__ q_out, const T* __restrict__ q, const T* __restrict__ k,
+    const T* __restrict__ v, long q_stride, long k_stride, long v_stride,
+    const long* __restrict__ pos, const double* __restrict__ inv_freq, int rot,
+    int pairs, int unit, float eps, int heads, int n_kv, int D, int Dv,
+    T* __restrict__ k_cache, T* __restrict__ v_cache,
+    const long* __restrict__ slot_mapping, int block_size, float mscale,
+    const float* __restrict__ wq, const float* __restrict__ wk,
+    const float* __restrict__ table) {
+  extern __shared__ float cs[];           // [rot/2] cos, [rot/2] sin
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const int half = rot >> 1;
+  if (table != nullptr) {
+    for (int i = tid; i < rot; i += 256) cs[i] = table[(long)t * rot + i];
+  } else {
+    for (int i = tid; i < half; i += 256) {
+      double s, c;
+      sincos((double)pos[t] * inv_freq[i], &s, &c);
+      cs[i] = (float)(c * mscale);
+      cs[half + i] = (float)(s * mscale);
+    }
+  }
+  __syncthreads();
+  const long slot = slot_mapping[t];
+  const long blk = slot >= 0 ? slot / block_size : 0;
+  const long off = slot >= 0 ? slot % block_size : 0;
+  const int units = k != nullptr && slot >= 0 ? heads + n_kv : heads;
+  const int gl = tid % LG, d = gl * 4;    // this lane's entries of its head
+  const bool on = d < D, turned = d < rot, first = pairs || d < half;
+  // whole groups run the same number of rounds (the exchanges need all lanes)
+  for (int u0 = 0; u0 < units; u0 += 256 / LG) {
+    const int u = u0 + tid / LG;
+    const bool live = on && u < units;
+    const bool is_q = u < heads;
+    float x[4] = {0.f, 0.f, 0.f, 0.f};
+    if (live)
+      Quad<T>::ld((is_q ? q + (long)t * q_stride + (long)u * D
+                        : k + (long)t * k_stride + (long)(u - heads) * D) + d,
+                  x);
+    const float* hw = is_q ? wq : wk;
+    if (wq != nullptr || wk != nullptr) {            // norm before the turn
+      const float ss = group_reduce_sum<LG>(x[0] * x[0] + x[1] * x[1] +
+                                            x[2] * x[2] + x[3] * x[3]);
+      if (hw != nullptr && live) {
+        const float rs = 1.0f / sqrtf(ss / (float)D + eps);
+        float w[4];
+        Quad<float>::ld(hw + d, w);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) x[j] = x[j] * rs * w[j];
+      }
+    }
+    if (rot > 0) {
+      float y[4], z[4];
+      if (pairs) {
+        y[0] = -x[1]; y[1] = x[0]; y[2] = -x[3]; y[3] = x[2];
+      } else {
+        const int from = (tid & ~(LG - 1) & 63) +
+                         (turned ? (first ? gl + (half >> 2)
+                                          : gl - (half >> 2)) : gl);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          z[j] = __shfl(x[j], from, 64);
+          y[j] = first ? -z[j] : z[j];
+        }
+      }
+      if (turned) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const int i = pairs ? (d + j) >> 1 : (first ? d : d - half) + j;
+          x[j] = x[j] * cs[i] + y[j] * cs[half + i];
+        }
+      }
+    }
+    if (unit) {
+      const float ss = group_reduce_sum<LG>(x[0] * x[0] + x[1] * x[1] +
+                                            x[2] * x[2] + x[3] * x[3]);
+      const float rs = 1.0f / sqrtf(ss / (float)D + eps);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) x[j] *= rs;
+    }
+    if (live)
+      Quad<T>::st((is_q ? q_out + ((long)t * heads + u) * D
+                        : k_cache + ((blk * n_kv + (u - heads)) * block_size +
+                                     off) * (long)D) + d, x);
+  }
+  if (v == nullptr || slot < 0) return;
+  const T* vr = v + (long)t * v_stride;
+  for (int i = tid; i < n_kv * Dv; i += 256) {
+    const int g = i / Dv, c = i - g * Dv;
+    v_cache[((blk * n_kv + g) * block_size + off) * (long)Dv + c] = vr[i];
+  }
+}
+
 template <typename T>
 __global__ void __launch_bounds__(256) polynorm_kernel(
     T* __restrict__ out, const T* __restrict__ z,
@@ -176,11 +275,28 @@ void launch_rope_headnorm_store(T* q_out, const T* q, const T* k, const T* v,
                                 const float* wk, const float* table,
                                 hipStream_t st) {
   if (tokens == 0) return;
-  hipLaunchKernelGGL((rope_headnorm_store_kernel<T>), dim3(tokens), dim3(256),
-                     (size_t)(rot > 0 ? rot : 1) * sizeof(float), st, q_out, q,
-                     k, v, q_stride, k_stride, v_stride, pos, inv_freq, rot,
-                     pairs, unit, eps, heads, n_kv, D, Dv, k_cache, v_cache,
-                     slot_mapping, block_size, mscale, wq, wk, table);
+  const size_t lds = (size_t)(rot > 0 ? rot : 1) * sizeof(float);
+#define RH_CALL(KERNEL)                                                       \
+  hipLaunchKernelGGL((KERNEL), dim3(tokens), dim3(256), lds, st, q_out, q, k, \
+                     v, q_stride, k_stride, v_stride, pos, inv_freq, rot,     \
+                     pairs, unit, eps, heads, n_kv, D, Dv, k_cache, v_cache,  \
+                     slot_mapping, block_size, mscale, wq, wk, table)
+  auto quads = [](const void* p, long stride, size_t size) {
+    return p == nullptr || (stride % 4 == 0 &&
+                            reinterpret_cast<uintptr_t>(p) % (4 * size) == 0);
+  };
+  if (D % 4 == 0 && D <= 256 && rot % (pairs ? 4 : 8) == 0 &&
+      quads(q, q_stride, sizeof(T)) && quads(k, k_stride, sizeof(T)) &&
+      quads(q_out, D, sizeof(T)) && quads(k_cache, D, sizeof(T)) &&
+      quads(wq, D, 4) && quads(wk, D, 4)) {
+    if (D <= 32) RH_CALL((rope_headnorm_quads_kernel<T, 8>));
+    else if (D <= 64) RH_CALL((rope_headnorm_quads_kernel<T, 16>));
+    else if (D <= 128) RH_CALL((rope_headnorm_quads_kernel<T, 32>));
+    else RH_CALL((rope_headnorm_quads_kernel<T, 64>));
+  } else {
+    RH_CALL((rope_headnorm_store_kernel<T>));
+  }
+#undef RH_CALL
 }
 
 template <typename T>
