@@ -257,3 +257,38 @@ def test_max_model_len_enforced():
     out = eng.generate([prompt], SamplingParams(max_tokens=64,
                                                 ignore_eos=True))[0]
     assert len(out) == 256 - 250                        # clamped to capacity
+
+
+def test_collector_rests_while_graphs_are_captured():
+    """Dead cycles go before a capture, none is collected during it, and the
+    collector is as it was afterwards, also after an error."""
+    import gc
+    import weakref
+
+    from xllm_service_amd.engine.graph_runner import collector_paused
+
+    class Node:
+        pass
+
+    def dead_cycle():
+        a = Node()
+        a.me = a
+        return weakref.ref(a)
+    before = dead_cycle()
+    with collector_paused():
+        assert before() is None and not gc.isenabled()
+        inside = dead_cycle()
+        junk = [[i] for i in range(200000)]        # would start a collection
+        assert inside() is not None and len(junk) == 200000
+    assert gc.isenabled()
+    with pytest.raises(RuntimeError):
+        with collector_paused():
+            raise RuntimeError("capture failed")
+    assert gc.isenabled()
+    gc.disable()
+    try:
+        with collector_paused():
+            pass
+        assert not gc.isenabled()
+    finally:
+        gc.enable()

@@ -9,6 +9,8 @@ point at block 0 with seq_len=16 so replays are always well-defined.
 """
 from __future__ import annotations
 
+import contextlib
+import gc
 import logging
 from typing import Dict, List, Optional, Tuple
 
@@ -39,6 +41,23 @@ def _mark_staging(pin: dict) -> None:
     ev.record()
 
 
+@contextlib.contextmanager
+def collector_paused():
+    """No cyclic garbage collection while a graph is being captured. Objects of
+    a dropped engine (graphs, events, pinned buffers) sit in reference cycles;
+    if the collector happens to run between two captured launches, their
+    destructors make HIP calls that a capturing thread may not make, and a
+    destructor that fails ends the process. What is already dead goes first."""
+    gc.collect()
+    was_on = gc.isenabled()
+    gc.disable()
+    try:
+        yield
+    finally:
+        if was_on:
+            gc.enable()
+
+
 class DecodeGraphRunner:
     def __init__(self, model, kv_caches, device, max_model_len: int = 4096,
                  max_batch: int = 256):
@@ -57,8 +76,9 @@ class DecodeGraphRunner:
         self._bt_rows: Dict[str, Tuple[np.ndarray, int]] = {}
 
     def capture_all(self):
-        for bs in sorted(self.buckets, reverse=True):  # largest first: pool
-            self._capture(bs)
+        with collector_paused():
+            for bs in sorted(self.buckets, reverse=True):  # largest first: pool
+                self._capture(bs)
         log.info("captured %d decode graphs (max_blocks=%d)",
                  len(self.graphs), self.max_blocks)
 
@@ -210,8 +230,9 @@ class PrefillGraphRunner:
         self._pinned: Dict[int, dict] = {}
 
     def capture_all(self):
-        for b in sorted(self.buckets, reverse=True):
-            self._capture(b)
+        with collector_paused():
+            for b in sorted(self.buckets, reverse=True):
+                self._capture(b)
         log.info("captured %d prefill graphs (buckets %s)",
                  len(self.graphs), self.buckets)
 
